@@ -136,17 +136,20 @@ int vla_seq_window_attention_tiles(void* out, int64_t out_stride, const void* q,
 #define VLA_ACT_GELU_TANH 4  /* 0.5 z (1 + tanh(sqrt(2/pi) (z + 0.044715 z^3))) */
 
 /* One launch around a sublayer, on the fp32 stream x [T, width] (in place):
- *   y given:        y' = y + y_bias (null: none);
- *                   x += y' / sqrt(mean(y'^2) + eps) * post_weight * layer_scale (layer_scale null: 1)
+ *   y given:        y' = y + y_bias (null: none);  u = y' / sqrt(mean(y'^2) + eps) * post_weight
+ *                   (post_weight null: u = y'), times layer_scale (null: 1);
+ *                   y2 given: u += y2 / sqrt(mean(y2^2) + eps) * post_weight2 (a second branch, not
+ *                   scaled by layer_scale);  x += u * y_scale
  *   add_row given:  x += add_row
  *   out given:      out = out_dtype(x / sqrt(mean(x^2) + eps) * pre_weight), or out_dtype(x) when
  *                   pre_weight is null
- * y is `y_dtype` rows of `width` values with stride y_stride; weights, layer_scale, add_row fp32
- * [width].  All of it fp32. */
+ * y and y2 are `y_dtype` rows of `width` values with strides y_stride / y2_stride; weights,
+ * layer_scale, add_row fp32 [width].  All of it fp32. */
 int vla_seq_residual_norms(float* x, const void* y, int64_t y_stride, int y_dtype,
                            const float* y_bias, const float* post_weight, const float* layer_scale,
                            const float* add_row, void* out, const float* pre_weight, float eps,
-                           int num_tokens, int width, int out_dtype, void* stream);
+                           int num_tokens, int width, int out_dtype, float y_scale, const void* y2,
+                           int64_t y2_stride, const float* post_weight2, void* stream);
 
 /* Causal convolution over time on each channel, added to its input:
  *   out[t] = dtype(h[t] + sum_j weight[:, j] h[t - taps + 1 + j]),  zeros before a sequence's start,
@@ -195,7 +198,8 @@ int vla_seq_pair_hash_embed(float* out, const void* table, const void* pair_tabl
  * are) turns the pairs of a value head over all vdim elements the same way.  Angles are fp32
  * products.  slot_mapping < 0 skips the caches.  q_norm [heads * dim] / k_norm [kv_heads * dim]
  * (fp32, null: none): the whole query / key row is divided by its root mean square (norm_eps inside
- * the root) and multiplied by these weights before it is rotated.  v_other (null: none; rows of
+ * the root) and multiplied by these weights before it is rotated; with head_norm every head is
+ * divided by its own root mean square over dim instead, and null weights mean 1.  v_other (null: none; rows of
  * kv_heads * vdim values, not together with value_inv_freq): the cached value is
  * (1 - v_blend[0]) v + v_blend[0] v_other, v_blend one fp32 number on the device. */
 int vla_seq_rotary_kv_write(void* q, int64_t q_stride, const void* k, int64_t k_stride,
@@ -206,13 +210,14 @@ int vla_seq_rotary_kv_write(void* q, int64_t q_stride, const void* k, int64_t k_
                             int interleaved, int block_size, int num_blocks, int dtype,
                             const float* q_norm, const float* k_norm, float norm_eps,
                             const void* v_other, int64_t v_other_stride, const float* v_blend,
-                            void* stream);
+                            int head_norm, void* stream);
 
 /* For the token at position p of sequence b and query head h (KV head h / (heads / kv_heads)):
- *   s_j = (q . k_j) * scale  for max(0, p - window + 1) <= j <= p  (window <= 0: all j <= p)
- *         and, with a window, for j < keep_first as well (a sequence's first tokens stay visible)
+ *   s_j = (q . k_j) * scale  for lo <= j <= p, lo = max(0, p - window + 1, p - p % chunk)
+ *         (window <= 0 / chunk <= 0: that bound is 0; chunks count from position 0) and, with a window
+ *         or a chunk, for j < keep_first as well (a sequence's first tokens stay visible)
  *   s_j <- softcap * tanh(s_j / softcap)                      (softcap 0: no cap)
- *   o = sum_j softmax(s)_j v_j;  out_inv_freq given: pair m of o turns by -p * out_inv_freq[m]
+ *   o = sum_j w_j v_j,  w_j = e^(s_j) / (sum_k e^(s_k) + e^(sinks[h]))   (sinks fp32 [heads]; null: softmax);  out_inv_freq given: pair m of o turns by -p * out_inv_freq[m]
  *   out = dtype(o * sigmoid(gate[t, h]))                      (gate null: no gate)
  * in fp32; the step's own keys and values must be in the caches already.  gate holds one number
  * per (token, head) with row stride gate_stride. */
@@ -222,7 +227,8 @@ int vla_seq_kv_attention(void* out, int64_t out_stride, const void* q, int64_t q
                          const int* token_seq, const int64_t* positions, const float* out_inv_freq,
                          int interleaved, int num_tokens, int heads, int kv_heads, int dim, int vdim,
                          int block_size, int num_blocks, int window, float scale, int dtype,
-                         int keep_first, float softcap, void* stream);
+                         int keep_first, float softcap, int chunk, const float* sinks,
+                         void* stream);
 
 /* The same attention for 16-bit activations, tiled over runs of 32 query rows of a sequence on
  * the matrix cores: rows query_start_loc[b] .. query_start_loc[b + 1] - 1 of sequence b sit at
@@ -238,7 +244,8 @@ int vla_seq_kv_attention_tiles(void* out, int64_t out_stride, const void* q, int
                                const float* out_inv_freq, int interleaved, int num_seqs,
                                int max_query_len, int heads, int kv_heads, int dim, int vdim,
                                int block_size, int num_blocks, int window, float scale, int dtype,
-                               int keep_first, float softcap, void* stream);
+                               int keep_first, float softcap, int chunk, const float* sinks,
+                               void* stream);
 int vla_seq_set_kv_attention_kernel(int mode);
 
 /* ---- element-wise gated recurrence (minGRU) ---------------------------------------------------- */
@@ -259,41 +266,46 @@ int vla_seq_mingru_scan(void* out, int64_t out_stride, const void* zp, int64_t z
 /* ---- mixture of experts in the activation dtype -------------------------------------------------- */
 
 /* Router of one token over `routed` experts (at most 512): z = router h + bias in fp32 (router
- * fp32 [routed, width], bias fp32 [routed] or null), s = softmax(z), the `top` largest s +
- * correction (null: s) are chosen, weights = their s / (sum + 1e-20) -- without a correction that
- * is the softmax over the chosen logits.  experts int32 / weights fp32 [T, top].  shared_gate given:
+ * fp32 [routed, width], bias fp32 [routed] or null), s = softmax(z) (score VLA_SCORE_SOFTMAX) or
+ * sigmoid(z) of each logit (VLA_SCORE_SIGMOID), the `top` largest s + correction (null: s) are
+ * chosen, weights = their s / (sum + 1e-20) with renormalize (softmax without a correction: the
+ * softmax over the chosen logits), their s as they are without.  experts int32 / weights fp32 [T, top].  shared_gate given:
  * shared_gate[t] = sigmoid(shared_gate_weight . h), shared_gate_weight fp32 [width].  logits given
  * (fp32 rows of routed (+ 1 with a shared gate, its logit last) values, stride logits_stride): the
  * products are the caller's and h, router, shared_gate_weight are not read. */
+#define VLA_SCORE_SOFTMAX 0
+#define VLA_SCORE_SIGMOID 1
 int vla_seq_moe_route(const void* h, int64_t h_stride, const float* router, const float* logits,
                       int64_t logits_stride, const float* bias, const float* correction,
                       const float* shared_gate_weight, int* experts, float* weights,
-                      float* shared_gate, int num_tokens, int width, int routed, int top, int dtype,
-                      void* stream);
+                      float* shared_gate, int num_tokens, int width, int routed, int top, int score,
+                      int renormalize, int dtype, void* stream);
 
 /* Groups the pairs (token, choice) whose expert is below num_experts by expert, every group padded
  * to whole tiles of vla_seq_moe_tile_rows() rows: pair_row int32 [T * top] (-1: the pair's expert
  * has no weights), row_token int32 [max_tiles * tile rows] (-1: padding), tile_expert int32
- * [max_tiles] (-1: unused).  max_tiles >= (T * top + (tile rows - 1) * min(num_experts, T * top))
+ * [max_tiles] (-1: unused).  weights and row_weight given (fp32, [T * top] and [max_tiles * tile
+ * rows]): row_weight[row] = the weight of the row's pair (padding: untouched).  max_tiles >= (T * top + (tile rows - 1) * min(num_experts, T * top))
  * / tile rows, rounded up, holds every case. */
 int vla_seq_moe_tile_rows(void);
 int vla_seq_moe_plan(const int* experts, int num_tokens, int top, int num_experts, int* pair_row,
-                     int* row_token, int* tile_expert, int max_tiles, void* stream);
+                     int* row_token, int* tile_expert, int max_tiles, const float* weights,
+                     float* row_weight, void* stream);
 
-/* out[row, :] = out_dtype(act(weight[e] a[src(row)])) for the rows of every tile, e =
+/* out[row, :] = out_dtype(act(weight[e] a[src(row)] * row_scale[row])) for the rows of every tile, e =
  * tile_expert[tile] (tiles with -1 are skipped), src(row) = row_token[row] (null: row; -1: a zero
- * row).  weight `dtype` [experts, n_out, k_in], a `dtype` rows of k_in values. */
+ * row), row_scale fp32 (null: 1; multiplies the fp32 sums: an expert whose input is weighted).  weight `dtype` [experts, n_out, k_in], a `dtype` rows of k_in values. */
 int vla_seq_grouped_linear(void* out, int64_t out_stride, int out_dtype, const void* a,
                            int64_t a_stride, const int* row_token, const void* weight,
                            const int* tile_expert, int max_tiles, int n_out, int k_in, int act,
-                           int dtype, void* stream);
+                           const float* row_scale, int dtype, void* stream);
 
 /* Form of the 16-bit product for tests: 0 = per shape, 1 = one-wave workgroups (decode steps),
  * 2 = runs of tiles per workgroup (prompts). */
 int vla_seq_set_grouped_linear_form(int mode);
 
 /* out[t] (fp32 [T, width]) = sum_k weights[t, k] * (y[pair_row[t, k]] or, where pair_row is -1,
- * h[t]) + shared_gate[t] * shared_y[t] (shared_y null: none; shared_gate null: 1).  y, shared_y
+ * h[t]) + shared_gate[t] * shared_y[t] (weights null: 1; shared_y null: none; shared_gate null: 1).  y, shared_y
  * fp32 rows of `width`. */
 int vla_seq_moe_combine(float* out, const float* y, const int* pair_row, const float* weights,
                         const void* h, int64_t h_stride, const float* shared_y,
@@ -363,6 +375,45 @@ int vla_seq_delta_rule_scan(void* out, int64_t out_stride, int out_dtype, const 
                             const int* context_lens, const int* state_slots, int num_tokens,
                             int num_seqs, int max_query_len, int num_slots, int heads, int kv_heads,
                             int dim, int vdim, float eps, float* scratch, void* stream);
+
+/* ---- linear recurrence with one decay per head and token -------------------------------------------- */
+
+/* Per head, on a state S [dim, vdim] in fp32:
+ *   S <- e^g S + w k v^T;   o = S^T q + skip v
+ * with q, k of the head's group (heads / groups heads share one query / key) and either
+ *   dt given:  w = softplus(dt row + dt_bias), g = -exp(a_log) w   (a state-space layer), or
+ *   dt null:   w = 1, g = log_decay[head]                          (constant decays).
+ * q, k and v pass `act` (VLA_ACT_NONE or VLA_ACT_SILU) first.  q, k [T, groups * dim],
+ * v [T, heads * vdim], dt [T, heads]: `dtype` rows with their own strides; dt_bias, a_log, log_decay,
+ * skip (null: none) fp32 [heads]; o fp32 [T, heads * vdim] contiguous; state fp32 [num_slots, heads,
+ * dim, vdim]; a sequence with context 0 starts from zero whatever its slot held.  Runs of more than
+ * VLA_DECAY_SCAN_PIECE rows are cut into pieces that are walked at once; scratch (fp32,
+ * vla_seq_decay_scan_scratch_floats values) holds their states.  max_query_len: the longest run of
+ * the step. */
+#define VLA_DECAY_SCAN_PIECE 256
+int64_t vla_seq_decay_scan_scratch_floats(int num_tokens, int num_seqs, int max_query_len, int heads,
+                                          int dim, int vdim);
+int vla_seq_decay_scan(float* o, const void* q, int64_t q_stride, const void* k, int64_t k_stride,
+                       const void* v, int64_t v_stride, const void* dt, int64_t dt_stride,
+                       const float* dt_bias, const float* a_log, const float* log_decay,
+                       const float* skip, float* state, const int* query_start_loc,
+                       const int* context_lens, const int* state_slots, int num_tokens, int num_seqs,
+                       int num_slots, int max_query_len, int heads, int groups, int dim, int vdim,
+                       int act, float* scratch, int64_t scratch_floats, int dtype, void* stream);
+/* Kernel choice for tests: 0 = per run of rows (runs of at most four token by token, longer ones in
+ * blocks on the matrix cores), 1 = always token by token, 2 = always in blocks. */
+int vla_seq_set_decay_scan_kernel(int mode);
+
+/* A recurrence's output rows o [T, n] (fp32, contiguous), gated and normed in `groups` equal parts
+ * (each by its own root mean square, eps inside the root):
+ *   gate_first:  u = o * gate_act(gate);  out = u / rms(u) * weight
+ *   otherwise:   out = o / rms(o) * weight * gate_act(gate)
+ * weight fp32 [n]; gate and out `dtype` rows of n values with their own strides. */
+#define VLA_GATE_SILU 0
+#define VLA_GATE_SIGMOID 1
+int vla_seq_gated_group_rms_norm(void* out, int64_t out_stride, const float* o, const float* weight,
+                                 const void* gate, int64_t gate_stride, int gate_act, int gate_first,
+                                 int groups, float eps, int num_tokens, int n, int dtype, void* stream);
 
 /* ---- real-gated linear recurrent unit ------------------------------------------------------------- */
 

@@ -259,29 +259,37 @@ def gla_combine_states(state: torch.Tensor, slots: torch.Tensor, pieces: torch.T
 
 # ---------------------------------------------------------------- layers with norms on both sides
 ACT = {"none": 0, "relu": 1, "relu2": 2, "silu": 3, "gelu_tanh": 4}
+MOE_SCORE = {"softmax": 0, "sigmoid": 1}
+GATE = {"silu": 0, "sigmoid": 1}
 
 
 def residual_norms(x: torch.Tensor, y: Optional[torch.Tensor] = None, y_bias: Optional[torch.Tensor] = None,
                    post_weight: Optional[torch.Tensor] = None,
                    layer_scale: Optional[torch.Tensor] = None, add_row: Optional[torch.Tensor] = None,
                    out: Optional[torch.Tensor] = None, pre_weight: Optional[torch.Tensor] = None,
-                   eps: float = 1e-5) -> None:
-    """x (fp32 [T, W], in place) += y' / rms(y') * post_weight * layer_scale with y' = y + y_bias;
-    x += add_row; out = x / rms(x) * pre_weight (pre_weight None: out = x).  Each part is optional."""
-    _gpu(x, y, y_bias, post_weight, layer_scale, add_row, out, pre_weight)
+                   eps: float = 1e-5, y_scale: float = 1.0, y2: Optional[torch.Tensor] = None,
+                   post_weight2: Optional[torch.Tensor] = None) -> None:
+    """x (fp32 [T, W], in place) += y_scale * (y' / rms(y') * post_weight * layer_scale + y2 / rms(y2) *
+    post_weight2) with y' = y + y_bias (post_weight None: y' as it is); x += add_row; out = x / rms(x)
+    * pre_weight (pre_weight None: out = x).  Each part is optional."""
+    _gpu(x, y, y_bias, post_weight, layer_scale, add_row, out, pre_weight, y2, post_weight2)
     T, W = x.shape
     assert x.dtype == torch.float32 and x.is_contiguous()
-    for v in (y_bias, post_weight, layer_scale, add_row, pre_weight):
+    for v in (y_bias, post_weight, layer_scale, add_row, pre_weight, post_weight2):
         assert v is None or (v.dtype == torch.float32 and v.numel() == W and v.is_contiguous())
     if y is not None:
-        assert y.shape == x.shape and post_weight is not None
+        assert y.shape == x.shape
+    if y2 is not None:
+        assert y is not None and y2.shape == x.shape and y2.dtype == y.dtype
+        assert post_weight is not None and post_weight2 is not None
     if out is not None:
         assert out.shape == x.shape and out.is_contiguous()
     with torch.cuda.device(x.device):
         seq_check(_lib.seq_lib().vla_seq_residual_norms(
             x.data_ptr(), _p(y), 0 if y is None else _rows(y, W), _lib.F32 if y is None else _dt(y.dtype),
             _p(y_bias), _p(post_weight), _p(layer_scale), _p(add_row), _p(out), _p(pre_weight), float(eps), T, W,
-            _lib.F32 if out is None else _dt(out.dtype), _stream(x.device)), "residual_norms")
+            _lib.F32 if out is None else _dt(out.dtype), float(y_scale), _p(y2), 0 if y2 is None else _rows(y2, W),
+            _p(post_weight2), _stream(x.device)), "residual_norms")
 
 
 def causal_conv(out: torch.Tensor, h: torch.Tensor, weight: torch.Tensor, state: Optional[torch.Tensor],
@@ -374,10 +382,12 @@ def rotary_kv_write(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, key_cache
                     inv_freq: Optional[torch.Tensor], value_inv_freq: Optional[torch.Tensor], heads: int,
                     rot_dims: int, interleaved: bool, q_norm: Optional[torch.Tensor] = None,
                     k_norm: Optional[torch.Tensor] = None, norm_eps: float = 0.0,
-                    v_other: Optional[torch.Tensor] = None, v_blend: Optional[torch.Tensor] = None) -> None:
+                    v_other: Optional[torch.Tensor] = None, v_blend: Optional[torch.Tensor] = None,
+                    head_norm: bool = False) -> None:
     """q [T, H*D] rotated in place; k [T, G*D], v [T, G*V] rotated into the caches
     [NB, BS, G, D] / [NB, BS, G, V].  q_norm fp32 [H*D] / k_norm fp32 [G*D]: the whole query / key
-    row is RMS-normed with these weights before the rotation.  v_other [T, G*V] with v_blend (fp32,
+    row is RMS-normed with these weights before the rotation; head_norm: every head by itself (no weights:
+    divided by its root mean square only).  v_other [T, G*V] with v_blend (fp32,
     one number on the device): the cached value is (1 - v_blend) v + v_blend v_other."""
     _gpu(q, k, v, key_cache, value_cache, positions, slot_mapping, inv_freq, value_inv_freq, q_norm, k_norm,
          v_other, v_blend)
@@ -403,17 +413,22 @@ def rotary_kv_write(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, key_cache
             key_cache.data_ptr(), value_cache.data_ptr(), positions.data_ptr(), slot_mapping.data_ptr(),
             _p(inv_freq), _p(value_inv_freq), T, heads, G, D, V, int(rot_dims), int(bool(interleaved)), BS, NB,
             _dt(q.dtype), _p(q_norm), _p(k_norm), float(norm_eps), _p(v_other),
-            0 if v_other is None else _rows(v_other, G * V), _p(v_blend), _stream(q.device)), "rotary_kv_write")
+            0 if v_other is None else _rows(v_other, G * V), _p(v_blend), int(bool(head_norm)), _stream(q.device)),
+            "rotary_kv_write")
 
 
 def kv_attention(out: torch.Tensor, q: torch.Tensor, gate: Optional[torch.Tensor], key_cache: torch.Tensor,
                  value_cache: torch.Tensor, block_tables: torch.Tensor, token_seq: torch.Tensor,
                  positions: torch.Tensor, out_inv_freq: Optional[torch.Tensor], interleaved: bool, heads: int,
-                 window: int, scale: float, keep_first: int = 0, softcap: float = 0.0) -> None:
+                 window: int, scale: float, keep_first: int = 0, softcap: float = 0.0, chunk: int = 0,
+                 sinks: Optional[torch.Tensor] = None) -> None:
     """out [T, H*V] = softmax attention of q [T, H*D] over the caches, output pairs turned back by
-    the position, times sigmoid(gate [T, H]).  With a window the first keep_first tokens of a
-    sequence stay visible; softcap > 0 caps the scores with softcap * tanh(score / softcap)."""
-    _gpu(out, q, gate, key_cache, value_cache, block_tables, token_seq, positions, out_inv_freq)
+    the position, times sigmoid(gate [T, H]).  With a window or a chunk the first keep_first tokens of a
+    sequence stay visible; softcap > 0 caps the scores with softcap * tanh(score / softcap); chunk > 0:
+    a row sees the keys of its own chunk of `chunk` positions only; sinks fp32 [H]: e^sinks joins a head's
+    softmax denominator."""
+    _gpu(out, q, gate, key_cache, value_cache, block_tables, token_seq, positions, out_inv_freq, sinks)
+    assert sinks is None or (sinks.dtype == torch.float32 and sinks.numel() == heads and sinks.is_contiguous())
     NB, BS, G, D = key_cache.shape
     V = value_cache.shape[3]
     T = q.shape[0]
@@ -432,7 +447,7 @@ def kv_attention(out: torch.Tensor, q: torch.Tensor, gate: Optional[torch.Tensor
             0 if gate is None else _rows(gate, heads), key_cache.data_ptr(), value_cache.data_ptr(),
             block_tables.data_ptr(), block_tables.shape[1], token_seq.data_ptr(), positions.data_ptr(),
             _p(out_inv_freq), int(bool(interleaved)), T, heads, G, D, V, BS, NB, int(window), float(scale),
-            _dt(q.dtype), int(keep_first), float(softcap), _stream(q.device)), "kv_attention")
+            _dt(q.dtype), int(keep_first), float(softcap), int(chunk), _p(sinks), _stream(q.device)), "kv_attention")
 
 
 def set_kv_attention_kernel(mode: int) -> None:
@@ -450,10 +465,11 @@ def kv_attention_tiles(out: torch.Tensor, q: torch.Tensor, gate: Optional[torch.
                        value_cache: torch.Tensor, block_tables: torch.Tensor, query_start_loc: torch.Tensor,
                        context_lens: torch.Tensor, max_query_len: int, out_inv_freq: Optional[torch.Tensor],
                        interleaved: bool, heads: int, window: int, scale: float, keep_first: int = 0,
-                       softcap: float = 0.0) -> None:
+                       softcap: float = 0.0, chunk: int = 0, sinks: Optional[torch.Tensor] = None) -> None:
     """The same attention as kv_attention for 16-bit activations, tiled over runs of 32 query rows
     of a sequence."""
-    _gpu(out, q, gate, key_cache, value_cache, block_tables, query_start_loc, context_lens, out_inv_freq)
+    _gpu(out, q, gate, key_cache, value_cache, block_tables, query_start_loc, context_lens, out_inv_freq, sinks)
+    assert sinks is None or (sinks.dtype == torch.float32 and sinks.numel() == heads and sinks.is_contiguous())
     NB, BS, G, D = key_cache.shape
     V = value_cache.shape[3]
     B = context_lens.numel()
@@ -472,7 +488,8 @@ def kv_attention_tiles(out: torch.Tensor, q: torch.Tensor, gate: Optional[torch.
             0 if gate is None else _rows(gate, heads), key_cache.data_ptr(), value_cache.data_ptr(),
             block_tables.data_ptr(), block_tables.shape[1], query_start_loc.data_ptr(), context_lens.data_ptr(),
             _p(out_inv_freq), int(bool(interleaved)), B, int(max_query_len), heads, G, D, V, BS, NB, int(window),
-            float(scale), _dt(q.dtype), int(keep_first), float(softcap), _stream(q.device)), "kv_attention_tiles")
+            float(scale), _dt(q.dtype), int(keep_first), float(softcap), int(chunk), _p(sinks), _stream(q.device)),
+            "kv_attention_tiles")
 
 
 def mingru_scan(out: torch.Tensor, zp: torch.Tensor, up: torch.Tensor, gp: torch.Tensor, state: torch.Tensor,
@@ -499,10 +516,11 @@ def mingru_scan(out: torch.Tensor, zp: torch.Tensor, up: torch.Tensor, gp: torch
 
 def moe_route(h: torch.Tensor, router: torch.Tensor, correction: Optional[torch.Tensor],
               shared_gate_weight: Optional[torch.Tensor], top: int, logits: Optional[torch.Tensor] = None,
-              bias: Optional[torch.Tensor] = None):
+              bias: Optional[torch.Tensor] = None, score: str = "softmax", renormalize: bool = True):
     """-> experts int32 [T, top], weights fp32 [T, top], shared gate fp32 [T] or None.  logits
     (fp32 [T, routed (+ 1, the shared gate's last)]): the router products, when the caller formed
-    them as one matrix product."""
+    them as one matrix product.  score: "softmax" over all experts or "sigmoid" of each logit; renormalize:
+    the chosen scores are divided by their sum."""
     _gpu(h, router, correction, shared_gate_weight, logits, bias)
     T, W = h.shape
     N = router.shape[0]
@@ -520,13 +538,14 @@ def moe_route(h: torch.Tensor, router: torch.Tensor, correction: Optional[torch.
         seq_check(_lib.seq_lib().vla_seq_moe_route(
             h.data_ptr(), _rows(h, W), router.data_ptr(), _p(logits), 0 if logits is None else logits.shape[1],
             _p(bias), _p(correction), _p(shared_gate_weight), experts.data_ptr(), weights.data_ptr(), _p(sg), T, W, N,
-            int(top), _dt(h.dtype), _stream(h.device)), "moe_route")
+            int(top), MOE_SCORE[score], int(bool(renormalize)), _dt(h.dtype), _stream(h.device)), "moe_route")
     return experts, weights, sg
 
 
-def moe_plan(experts: torch.Tensor, num_experts: int):
-    """-> pair_row int32 [T, top], row_token int32 [rows], tile_expert int32 [tiles]."""
-    _gpu(experts)
+def moe_plan(experts: torch.Tensor, num_experts: int, weights: Optional[torch.Tensor] = None):
+    """-> pair_row int32 [T, top], row_token int32 [rows], tile_expert int32 [tiles]; with weights (fp32
+    [T, top]) also row_weight fp32 [rows], the weight of each row's pair (padding rows: anything)."""
+    _gpu(experts, weights)
     T, top = experts.shape
     L = _lib.seq_lib()
     tile = L.vla_seq_moe_tile_rows()
@@ -535,17 +554,22 @@ def moe_plan(experts: torch.Tensor, num_experts: int):
     row_token = torch.empty((max_tiles * tile, ), dtype=torch.int32, device=experts.device)
     tile_expert = torch.empty((max_tiles, ), dtype=torch.int32, device=experts.device)
     assert experts.dtype == torch.int32 and experts.is_contiguous()
+    row_weight = None
+    if weights is not None:
+        assert weights.dtype == torch.float32 and weights.is_contiguous() and weights.shape == experts.shape
+        row_weight = torch.empty((max_tiles * tile, ), dtype=torch.float32, device=experts.device)
     with torch.cuda.device(experts.device):
         seq_check(L.vla_seq_moe_plan(experts.data_ptr(), T, top, int(num_experts), pair_row.data_ptr(),
-                                     row_token.data_ptr(), tile_expert.data_ptr(), max_tiles,
-                                     _stream(experts.device)), "moe_plan")
-    return pair_row, row_token, tile_expert
+                                     row_token.data_ptr(), tile_expert.data_ptr(), max_tiles, _p(weights),
+                                     _p(row_weight), _stream(experts.device)), "moe_plan")
+    return (pair_row, row_token, tile_expert) if weights is None else (pair_row, row_token, tile_expert, row_weight)
 
 
 def grouped_linear(out: torch.Tensor, a: torch.Tensor, row_token: Optional[torch.Tensor], weight: torch.Tensor,
-                   tile_expert: torch.Tensor, act: str = "none") -> None:
-    """out [tiles * tile rows, N] = act(weight[e] a[src(row)]); weight [E, N, K]; a rows of K."""
-    _gpu(out, a, row_token, weight, tile_expert)
+                   tile_expert: torch.Tensor, act: str = "none", row_scale: Optional[torch.Tensor] = None) -> None:
+    """out [tiles * tile rows, N] = act(weight[e] a[src(row)] * row_scale[row]); weight [E, N, K]; a rows
+    of K; row_scale fp32 per row (None: 1)."""
+    _gpu(out, a, row_token, weight, tile_expert, row_scale)
     E, N, K = weight.shape
     assert weight.is_contiguous() and weight.dtype == a.dtype and a.shape[1] == K
     L = _lib.seq_lib()
@@ -554,10 +578,12 @@ def grouped_linear(out: torch.Tensor, a: torch.Tensor, row_token: Optional[torch
     assert row_token is None or (row_token.dtype == torch.int32 and row_token.numel() == out.shape[0])
     if row_token is None:
         assert a.shape[0] == out.shape[0]
+    assert row_scale is None or (row_scale.dtype == torch.float32 and row_scale.numel() == out.shape[0])
     with torch.cuda.device(a.device):
         seq_check(L.vla_seq_grouped_linear(
             out.data_ptr(), N, _dt(out.dtype), a.data_ptr(), _rows(a, K), _p(row_token), weight.data_ptr(),
-            tile_expert.data_ptr(), tiles, N, K, ACT[act], _dt(a.dtype), _stream(a.device)), "grouped_linear")
+            tile_expert.data_ptr(), tiles, N, K, ACT[act], _p(row_scale), _dt(a.dtype), _stream(a.device)),
+            "grouped_linear")
 
 
 def set_grouped_linear_form(mode: int) -> None:
@@ -565,7 +591,7 @@ def set_grouped_linear_form(mode: int) -> None:
     seq_check(_lib.seq_lib().vla_seq_set_grouped_linear_form(mode), "set_grouped_linear_form")
 
 
-def moe_combine(out: torch.Tensor, y: torch.Tensor, pair_row: torch.Tensor, weights: torch.Tensor,
+def moe_combine(out: torch.Tensor, y: torch.Tensor, pair_row: torch.Tensor, weights: Optional[torch.Tensor],
                 h: torch.Tensor, shared_y: Optional[torch.Tensor], shared_gate: Optional[torch.Tensor]) -> None:
     _gpu(out, y, pair_row, weights, h, shared_y, shared_gate)
     T, W = h.shape
@@ -575,7 +601,7 @@ def moe_combine(out: torch.Tensor, y: torch.Tensor, pair_row: torch.Tensor, weig
     assert shared_y is None or (shared_y.dtype == torch.float32 and shared_y.is_contiguous() and shared_y.shape == (T, W))
     with torch.cuda.device(h.device):
         seq_check(_lib.seq_lib().vla_seq_moe_combine(
-            out.data_ptr(), y.data_ptr(), pair_row.data_ptr(), weights.data_ptr(), h.data_ptr(), _rows(h, W),
+            out.data_ptr(), y.data_ptr(), pair_row.data_ptr(), _p(weights), h.data_ptr(), _rows(h, W),
             _p(shared_y), _p(shared_gate), T, W, top, _dt(h.dtype), _stream(h.device)), "moe_combine")
 
 
@@ -704,6 +730,61 @@ def delta_rule_scan(out: torch.Tensor, q: torch.Tensor, k: torch.Tensor, v: torc
 def set_delta_kernel(mode: int) -> None:
     """0: delta_rule_scan picks its kernel per step; 1: always the one without staging; 2: never."""
     seq_check(_lib.seq_lib().vla_seq_set_delta_kernel(mode), "set_delta_kernel")
+
+
+# ---------------------------------------------------------------- recurrences with one decay per head
+def decay_scan(o: torch.Tensor, q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, state: torch.Tensor,
+               query_start_loc: torch.Tensor, context_lens: torch.Tensor, state_slots: torch.Tensor, groups: int,
+               max_query_len: int, log_decay: Optional[torch.Tensor] = None, dt: Optional[torch.Tensor] = None,
+               dt_bias: Optional[torch.Tensor] = None, a_log: Optional[torch.Tensor] = None,
+               skip: Optional[torch.Tensor] = None, act: str = "none") -> None:
+    """Per head S <- e^g S + w k v^T, o = S^T q + skip v; g = log_decay[h] and w = 1, or w = softplus(dt +
+    dt_bias) and g = -exp(a_log) w; q, k, v pass `act` ("none" or "silu") first.  o fp32 [T, H*V];
+    q, k [T, groups*D], v [T, H*V], dt [T, H]: views with free row strides; log_decay, dt_bias, a_log,
+    skip fp32 [H]; state fp32 [slots, H, D, V]."""
+    _gpu(o, q, k, v, state, query_start_loc, context_lens, state_slots, log_decay, dt, dt_bias, a_log, skip)
+    slots, H, D, V = state.shape
+    T, B = q.shape[0], context_lens.numel()
+    assert o.dtype == torch.float32 and o.is_contiguous() and o.shape == (T, H * V)
+    assert state.dtype == torch.float32 and state.is_contiguous()
+    assert q.dtype == k.dtype == v.dtype and (dt is None or dt.dtype == q.dtype)
+    assert (dt is None) != (log_decay is None) and (dt is None or (dt_bias is not None and a_log is not None))
+    for t in (log_decay, dt_bias, a_log, skip):
+        assert t is None or (t.dtype == torch.float32 and t.numel() == H and t.is_contiguous())
+    for t in (query_start_loc, context_lens, state_slots):
+        assert t.dtype == torch.int32 and t.is_contiguous()
+    assert query_start_loc.numel() == B + 1 and state_slots.numel() == B
+    L = _lib.seq_lib()
+    need = L.vla_seq_decay_scan_scratch_floats(T, B, int(max_query_len), H, D, V)
+    scratch = torch.empty(need, dtype=torch.float32, device=q.device) if need else None
+    with torch.cuda.device(q.device):
+        seq_check(L.vla_seq_decay_scan(
+            o.data_ptr(), q.data_ptr(), _rows(q, groups * D), k.data_ptr(), _rows(k, groups * D), v.data_ptr(),
+            _rows(v, H * V), _p(dt), 0 if dt is None else _rows(dt, H), _p(dt_bias), _p(a_log), _p(log_decay),
+            _p(skip), state.data_ptr(), query_start_loc.data_ptr(), context_lens.data_ptr(), state_slots.data_ptr(),
+            T, B, slots, int(max_query_len), H, int(groups), D, V, ACT[act], _p(scratch), need, _dt(q.dtype),
+            _stream(q.device)), "decay_scan")
+
+
+def set_decay_scan_kernel(mode: int) -> None:
+    """0: decay_scan picks its kernel per run of rows; 1: always token by token; 2: always in blocks."""
+    seq_check(_lib.seq_lib().vla_seq_set_decay_scan_kernel(mode), "set_decay_scan_kernel")
+
+
+def gated_group_rms_norm(out: torch.Tensor, o: torch.Tensor, weight: torch.Tensor, gate: torch.Tensor, gate_act: str,
+                         gate_first: bool, groups: int, eps: float) -> None:
+    """gate_first: u = o * gate_act(gate), out = u / rms(u) * weight; else out = o / rms(o) * weight *
+    gate_act(gate); the norm runs over each of `groups` equal parts of a row.  o fp32 [T, n]; gate, out
+    [T, n] views with free row strides; gate_act "silu" or "sigmoid"."""
+    _gpu(out, o, weight, gate)
+    T, n = o.shape
+    assert o.dtype == torch.float32 and o.is_contiguous() and out.dtype == gate.dtype
+    assert weight.dtype == torch.float32 and weight.numel() == n and weight.is_contiguous()
+    with torch.cuda.device(o.device):
+        seq_check(_lib.seq_lib().vla_seq_gated_group_rms_norm(
+            out.data_ptr(), _rows(out, n), o.data_ptr(), weight.data_ptr(), gate.data_ptr(), _rows(gate, n),
+            GATE[gate_act], int(bool(gate_first)), int(groups), float(eps), T, n, _dt(out.dtype), _stream(o.device)),
+            "gated_group_rms_norm")
 
 
 def rglru_scan(out: torch.Tensor, gates: torch.Tensor, u: torch.Tensor, y: torch.Tensor,

@@ -10,7 +10,9 @@ distance.  An optional window keeps 0 <= i - j < window, and with `keep_first` a
 keep_first (a sequence's first tokens stay visible, at their true positions); `softcap` replaces a
 score s by softcap * tanh(s / softcap); `freq_scale` divides every rotary frequency (linear position
 scaling); `norm_rows` norms the whole query row and the whole key row (all heads at once, RMS with
-a weight per element) before the rotation; an optional gate multiplies each head's output by the
+a weight per element) before the rotation, `norm_heads` every head by itself (no weight); `chunk` lets
+position i see only the keys of its own chunk of `chunk` positions (counted from position 0);
+`sink_score` adds e^sink_score to every head's softmax denominator (a key without a value); an optional gate multiplies each head's output by the
 sigmoid of one number per (token, head); forward's `v_other` / `v_blend` cache
 (1 - v_blend) v + v_blend v_other instead of v (values blended with another layer's values of the
 same tokens).  Every parameter is a constructor argument.  Prompts, portions of prompts and decode steps are one case: the step's keys and values
@@ -42,12 +44,17 @@ class RotaryKVAttention(nn.Module):
     def __init__(self, num_heads: int, num_kv_heads: int, head_dim: int, value_dim: int, scale: float,
                  rot_dims: int, rot_base: float, interleaved: bool = True, rotate_values: bool = False,
                  window: Optional[int] = None, device=None, keep_first: int = 0, softcap: float = 0.0,
-                 freq_scale: float = 1.0, norm_rows: bool = False, norm_eps: float = 1e-5) -> None:
+                 freq_scale: float = 1.0, norm_rows: bool = False, norm_eps: float = 1e-5, norm_heads: bool = False,
+                 chunk: Optional[int] = None, sink_score: Optional[float] = None) -> None:
         super().__init__()
         assert num_heads % num_kv_heads == 0 and 0 <= rot_dims <= head_dim and rot_dims % 2 == 0
         assert not rotate_values or value_dim % 2 == 0
-        assert keep_first >= 0 and softcap >= 0.0 and freq_scale > 0.0
-        self.keep_first = int(keep_first) if window else 0
+        assert keep_first >= 0 and softcap >= 0.0 and freq_scale > 0.0 and not (norm_rows and norm_heads)
+        self.chunk, self.norm_heads = int(chunk) if chunk else 0, bool(norm_heads)
+        self.keep_first = int(keep_first) if window or chunk else 0
+        self.register_buffer("sinks", None if sink_score is None else
+                             torch.full((num_heads, ), float(sink_score), dtype=torch.float32, device=device),
+                             persistent=False)
         self.softcap, self.norm_eps = float(softcap), float(norm_eps)
         self.q_norm = nn.Parameter(torch.ones(num_heads * head_dim, dtype=torch.float32, device=device),
                                    requires_grad=False) if norm_rows else None
@@ -80,16 +87,17 @@ class RotaryKVAttention(nn.Module):
         ops.rotary_kv_write(q, k, v, key_cache, value_cache, batch.positions, batch.slot_mapping,
                             self.inv_freq, self.value_inv_freq, self.num_heads, self.rot_dims, self.interleaved,
                             None if self.q_norm is None else self.q_norm.data,
-                            None if self.k_norm is None else self.k_norm.data, self.norm_eps, v_other, v_blend)
+                            None if self.k_norm is None else self.k_norm.data, self.norm_eps, v_other, v_blend,
+                            self.norm_heads)
         if batch.max_query_len >= self.TILE_MIN_QUERY and \
                 ops.kv_attention_tiles_supported(q, self.head_dim, self.value_dim):
             # a step with runs of rows (prompts, portions): 32-row tiles on the matrix cores
             ops.kv_attention_tiles(out, q, gate, key_cache, value_cache, batch.block_tables,
                                    batch.query_start_loc, batch.context_lens, batch.max_query_len,
                                    self.value_inv_freq, self.interleaved, self.num_heads, self.window, self.scale,
-                                   self.keep_first, self.softcap)
+                                   self.keep_first, self.softcap, self.chunk, self.sinks)
         else:
             ops.kv_attention(out, q, gate, key_cache, value_cache, batch.block_tables, batch.token_seq,
                              batch.positions, self.value_inv_freq, self.interleaved, self.num_heads, self.window,
-                             self.scale, self.keep_first, self.softcap)
+                             self.scale, self.keep_first, self.softcap, self.chunk, self.sinks)
         return out

@@ -13,14 +13,16 @@ product (o_t += (q_t exp(c_t))^T S_start, c_t the log decays summed from the pie
 and the pieces' states are chained by a cheap walk.  The result is the long walk's, to rounding.
 Kernels: csrc/seq_linear_recurrence.hip, csrc/seq_stream_kernels.hip.
 """
+import math
 import os
-from typing import Optional, Tuple
+from typing import Optional, Sequence, Tuple
 
 import torch
 import torch.nn as nn
 
 from vllm_legacy_amd import _seq_ops as ops
 from vllm_legacy_amd.attention.batch import SequenceBatch
+from vllm_legacy_amd.layers import ShortConv
 
 
 class GatedLinearRecurrence(nn.Module):
@@ -228,4 +230,82 @@ class RealGatedLRU(nn.Module):
         gates = torch.baddbmm(self.gate_bias.data, u.view(T, B, bw).transpose(0, 1), self.gate_weight.data)
         ops.rglru_scan(out, gates, u, y, self.rate.data, state, batch.query_start_loc, batch.context_lens,
                        batch.state_slots, batch.max_query_len)
+        return out
+
+
+class ConstantDecayRecurrence(nn.Module):
+    """Linear attention with one constant decay per head and per-sequence state slots:
+    S_t = decay_h S_(t-1) + k_t v_t^T, o_t = S_t^T q_t with q, k, v = act of their projections; the
+    concatenated heads are RMS-normed together with a weight per element and multiplied by
+    sigmoid(gate).  The state is fp32 [num_slots, heads, dim, vdim] and a sequence whose context length
+    is 0 starts from zero whatever its slot held (csrc/seq_decay_scan.hip)."""
+
+    def __init__(self, heads: int, dim: int, vdim: int, decay: Sequence[float], eps: float, act: str = "silu",
+                 device=None) -> None:
+        super().__init__()
+        if len(decay) != heads or not all(0.0 <= float(d) <= 1.0 for d in decay):
+            raise ValueError("one decay in [0, 1] per head is needed")
+        self.heads, self.dim, self.vdim, self.eps, self.act = heads, dim, vdim, float(eps), act
+        # a decay of 0 forgets everything: a finite stand-in for its logarithm keeps sums of it finite
+        logs = [max(math.log(d), -1e30) if d > 0.0 else -1e30 for d in map(float, decay)]
+        self.register_buffer("log_decay", torch.tensor(logs, dtype=torch.float64).to(torch.float32).to(device),
+                             persistent=False)
+        self.norm_weight = nn.Parameter(torch.ones(heads * vdim, dtype=torch.float32, device=device), requires_grad=False)
+
+    @staticmethod
+    def get_state_shape(num_slots: int, heads: int, dim: int, vdim: int) -> Tuple[int, ...]:
+        return (num_slots, heads, dim, vdim)
+
+    def forward(self, out: torch.Tensor, q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, gate: torch.Tensor,
+                state: torch.Tensor, batch: SequenceBatch) -> torch.Tensor:
+        """q, k [T, H*D]; v, gate, out [T, H*V]: views with free row strides, before their activations."""
+        o = torch.empty((q.shape[0], self.heads * self.vdim), dtype=torch.float32, device=q.device)
+        ops.decay_scan(o, q, k, v, state, batch.query_start_loc, batch.context_lens, batch.state_slots, self.heads,
+                       batch.max_query_len, log_decay=self.log_decay, act=self.act)
+        ops.gated_group_rms_norm(out, o, self.norm_weight.data, gate, "sigmoid", False, 1, self.eps)
+        return out
+
+
+class StateSpaceRecurrence(nn.Module):
+    """State-space layer with a scalar decay per head and token (state-space duality).  The projection's
+    rows are [z | x | B | C | dt]; x, B and C pass a causal convolution over time per channel with a bias
+    and silu (its last inputs live in a state slot of their own); with step = softplus(dt + dt_bias),
+    S_t = exp(-exp(a_log) step) S_(t-1) + step B_t x_t^T and y_t = S_t^T C_t + D x_t per head (heads /
+    groups heads share B and C), S [state, vdim] fp32; y silu(z) leaves RMS-normed in norm_groups equal
+    parts with a weight per element.  A sequence whose context length is 0 starts from zero whatever its
+    slots held (csrc/seq_decay_scan.hip, csrc/seq_post_norm_kernels.hip)."""
+
+    def __init__(self, heads: int, vdim: int, state: int, groups: int, norm_groups: int, taps: int, eps: float,
+                 device=None) -> None:
+        super().__init__()
+        inner = heads * vdim
+        if heads % groups or inner % norm_groups:
+            raise ValueError("heads must divide into the groups and their outputs into the norm's parts")
+        self.heads, self.vdim, self.state, self.groups, self.norm_groups = heads, vdim, state, groups, norm_groups
+        self.inner, self.eps = inner, float(eps)
+        self.channels = inner + 2 * groups * state
+        self.conv = ShortConv(self.channels, taps, True, "silu", device)
+
+        def par(n, fill=0.0):
+            return nn.Parameter(torch.full((n, ), fill, dtype=torch.float32, device=device), requires_grad=False)
+
+        self.a_log, self.dt_bias, self.skip, self.norm_weight = par(heads), par(heads), par(heads, 1.0), par(inner, 1.0)
+
+    @staticmethod
+    def get_state_shapes(num_slots: int, heads: int, vdim: int, state: int, groups: int,
+                         taps: int) -> Tuple[Tuple[int, ...], Tuple[int, ...]]:
+        """(recurrent state, the convolution's last inputs)."""
+        return ((num_slots, heads, state, vdim), ShortConv.get_state_shape(num_slots, heads * vdim + 2 * groups * state, taps))
+
+    def forward(self, out: torch.Tensor, z: torch.Tensor, xbc: torch.Tensor, dt: torch.Tensor, state: torch.Tensor,
+                conv_state: Optional[torch.Tensor], batch: SequenceBatch) -> torch.Tensor:
+        """z, out [T, inner], xbc [T, channels], dt [T, heads]: views with free row strides."""
+        T, inner, gn = z.shape[0], self.inner, self.groups * self.state
+        u = torch.empty((T, self.channels), dtype=z.dtype, device=z.device)
+        self.conv(u, xbc, conv_state, batch)
+        y = torch.empty((T, inner), dtype=torch.float32, device=z.device)
+        ops.decay_scan(y, u[:, inner + gn:], u[:, inner:inner + gn], u[:, :inner], state, batch.query_start_loc,
+                       batch.context_lens, batch.state_slots, self.groups, batch.max_query_len, dt=dt,
+                       dt_bias=self.dt_bias.data, a_log=self.a_log.data, skip=self.skip.data)
+        ops.gated_group_rms_norm(out, y, self.norm_weight.data, z, "silu", True, self.norm_groups, self.eps)
         return out

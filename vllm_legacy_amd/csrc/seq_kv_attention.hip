@@ -1,12 +1,14 @@
 // Causal softmax attention over paged key and value caches with rotary positions on queries and
 // keys, values that are rotated by their own position when they are cached (the head's output is
 // turned back by the query's position), an optional sliding window that may keep a sequence's
-// first tokens visible, an optional cap on the scores (cap * tanh(score / cap)) and a sigmoid gate of
-// one number per head.  rotary_kv_write can also norm the whole query and key rows before it rotates
-// them and blend the values with another layer's values of the same tokens.
+// first tokens visible, optional chunks (a row sees the keys of its own chunk of positions only), an
+// optional cap on the scores (cap * tanh(score / cap)), an optional sink per head (one more term in the
+// softmax denominator that has no value) and a sigmoid gate of one number per head.  rotary_kv_write
+// can also norm the whole query and key rows, or every head, before it rotates them and blend the
+// values with another layer's values of the same tokens.
 //
 // With a window and `keep_first` kept tokens, query position p sees j <= p with p - j < window or
-// j < keep_first.  The kernels walk such a key set through one index u: with lo the window's first
+// j < keep_first; with chunks, j >= p - p % chunk (both: the later of the two bounds).  The kernels walk such a key set through one index u: with lo the window's first
 // key and nk = min(keep_first, lo), u < nk is key u and u >= nk is key lo + u - nk.
 //
 // Caches: keys [num_blocks, block_size, kv_heads, dim] and values [num_blocks, block_size, kv_heads,
@@ -48,6 +50,14 @@ __device__ __forceinline__ float cap_score_fast(float s, float cap, float two_lo
   return cap - 2.f * cap * __builtin_amdgcn_rcpf(e + 1.f);
 }
 
+// the first key position p sees (kept tokens apart): its window's, or its chunk's, whichever is later;
+// never decreases with p
+__device__ __forceinline__ int first_key(int p, int window, int chunk) {
+  int lo = window > 0 ? max(0, p - window + 1) : 0;
+  if (chunk > 0) lo = max(lo, p - p % chunk);
+  return lo;
+}
+
 // element indices of pair i among `span` rotated elements
 __device__ __forceinline__ void pair_index(int i, int span, int interleaved, int& ia, int& ib) {
   if (interleaved) {
@@ -70,8 +80,9 @@ __global__ __launch_bounds__(256) void rotary_kv_write_kernel(
     int kv_heads, int dim, int vdim, int rot_dims, int interleaved, int64_t num_slots,
     const float* __restrict__ q_norm, const float* __restrict__ k_norm, float norm_eps,
     const typename S::T* __restrict__ v_other, int64_t v_other_stride,
-    const float* __restrict__ v_blend) {
+    const float* __restrict__ v_blend, int head_norm) {
   using T = typename S::T;
+  extern __shared__ float head_inv[];     // head_norm: 1 / rms of every query head, then of every key head
   __shared__ float red[16];
   const int t = blockIdx.x;
   const float p = (float)positions[t];
@@ -83,7 +94,31 @@ __global__ __launch_bounds__(256) void rotary_kv_write_kernel(
   const T* kr = k + (int64_t)t * k_stride;
   // RMS norm over the whole row (all heads at once) with a weight per element, before the rotation
   float q_inv = 1.f, k_inv = 1.f;
-  if (q_norm != nullptr) {
+  if (head_norm) {
+    // a quarter wave per head
+    const int sub = threadIdx.x & 15;
+    for (int h = threadIdx.x >> 4; h < heads + kv_heads; h += 16) {
+      const T* hr = h < heads ? qr + h * dim : kr + (h - heads) * dim;
+      float ss = 0.f;
+      for (int d = sub; d < dim; d += 16) {
+        const float x = S::to_f32(hr[d]);
+        ss += x * x;
+      }
+#pragma unroll
+      for (int m = 8; m >= 1; m >>= 1) ss += __shfl_xor(ss, m, 16);
+      if (sub == 0) head_inv[h] = 1.f / sqrtf(ss / (float)dim + norm_eps);
+    }
+    __syncthreads();
+  }
+  // factor of element i of query / key head h
+  auto q_factor = [&](int h, int i) {
+    return (head_norm ? head_inv[h] : q_inv) * (q_norm != nullptr ? q_norm[h * dim + i] : 1.f);
+  };
+  auto k_factor = [&](int h, int i) {
+    return (head_norm ? head_inv[heads + h] : k_inv) * (k_norm != nullptr ? k_norm[h * dim + i] : 1.f);
+  };
+  const bool q_normed = head_norm || q_norm != nullptr, k_normed = head_norm || k_norm != nullptr;
+  if (!head_norm && q_norm != nullptr) {
     float ss = 0.f;
     for (int i = threadIdx.x; i < heads * dim; i += blockDim.x) {
       const float x = S::to_f32(qr[i]);
@@ -91,7 +126,7 @@ __global__ __launch_bounds__(256) void rotary_kv_write_kernel(
     }
     q_inv = 1.f / sqrtf(block_sum(ss, red) / (float)(heads * dim) + norm_eps);
   }
-  if (k_norm != nullptr) {
+  if (!head_norm && k_norm != nullptr) {
     float ss = 0.f;
     for (int i = threadIdx.x; i < kv_heads * dim; i += blockDim.x) {
       const float x = S::to_f32(kr[i]);
@@ -104,18 +139,18 @@ __global__ __launch_bounds__(256) void rotary_kv_write_kernel(
     int ia, ib;
     pair_index(f, rot_dims, interleaved, ia, ib);
     float a = S::to_f32(qr[h * dim + ia]), b = S::to_f32(qr[h * dim + ib]);
-    if (q_norm != nullptr) {
-      a *= q_inv * q_norm[h * dim + ia];
-      b *= q_inv * q_norm[h * dim + ib];
+    if (q_normed) {
+      a *= q_factor(h, ia);
+      b *= q_factor(h, ib);
     }
     turn(a, b, p * inv_freq[f]);
     qr[h * dim + ia] = S::from_f32(a);
     qr[h * dim + ib] = S::from_f32(b);
   }
-  if (q_norm != nullptr) {
+  if (q_normed) {
     for (int i = threadIdx.x; i < heads * rest; i += blockDim.x) {
       const int h = i / rest, d = rot_dims + (i - h * rest);
-      qr[h * dim + d] = S::from_f32(S::to_f32(qr[h * dim + d]) * q_inv * q_norm[h * dim + d]);
+      qr[h * dim + d] = S::from_f32(S::to_f32(qr[h * dim + d]) * q_factor(h, d));
     }
   }
   if (!cached) return;
@@ -125,9 +160,9 @@ __global__ __launch_bounds__(256) void rotary_kv_write_kernel(
     int ia, ib;
     pair_index(f, rot_dims, interleaved, ia, ib);
     float a = S::to_f32(kr[h * dim + ia]), b = S::to_f32(kr[h * dim + ib]);
-    if (k_norm != nullptr) {
-      a *= k_inv * k_norm[h * dim + ia];
-      b *= k_inv * k_norm[h * dim + ib];
+    if (k_normed) {
+      a *= k_factor(h, ia);
+      b *= k_factor(h, ib);
     }
     turn(a, b, p * inv_freq[f]);
     kc[h * dim + ia] = S::from_f32(a);
@@ -135,8 +170,8 @@ __global__ __launch_bounds__(256) void rotary_kv_write_kernel(
   }
   for (int i = threadIdx.x; i < kv_heads * rest; i += blockDim.x) {
     const int h = i / rest, d = rot_dims + (i - h * rest);
-    if (k_norm != nullptr)
-      kc[h * dim + d] = S::from_f32(S::to_f32(kr[h * dim + d]) * k_inv * k_norm[h * dim + d]);
+    if (k_normed)
+      kc[h * dim + d] = S::from_f32(S::to_f32(kr[h * dim + d]) * k_factor(h, d));
     else
       kc[h * dim + d] = kr[h * dim + d];
   }
@@ -209,7 +244,7 @@ __global__ __launch_bounds__(kWave* kHeadsPerGroup) void kv_attention_kernel(
     const int* __restrict__ block_tables, int max_blocks, const int* __restrict__ token_seq,
     const int64_t* __restrict__ positions, const float* __restrict__ out_inv_freq, int interleaved,
     int heads, int kv_heads, int dim, int vdim, int block_size, int num_blocks, int window,
-    float scale, int keep_first, float softcap) {
+    float scale, int keep_first, float softcap, int chunk, const float* __restrict__ sinks) {
   __shared__ float q_lds[kHeadsPerGroup][kMaxDim];
   __shared__ float p_lds[kHeadsPerGroup][kWave];
   const int lane = threadIdx.x & 63, w = threadIdx.x >> 6;
@@ -219,7 +254,7 @@ __global__ __launch_bounds__(kWave* kHeadsPerGroup) void kv_attention_kernel(
   const int g = h / (heads / kv_heads);
   const int p = (int)positions[t];
   const int* table = block_tables + (int64_t)token_seq[t] * max_blocks;
-  const int lo = window > 0 ? max(0, p - window + 1) : 0;
+  const int lo = first_key(p, window, chunk);
   const int nk = min(keep_first, lo);         // kept keys ahead of the window
   const int total = nk + p - lo + 1;
   auto key_of = [&](int u) { return u < nk ? u : u - nk + lo; };
@@ -236,7 +271,8 @@ __global__ __launch_bounds__(kWave* kHeadsPerGroup) void kv_attention_kernel(
   float acc[kAccum];
 #pragma unroll
   for (int c = 0; c < kAccum; ++c) acc[c] = 0.f;
-  float m = -INFINITY, l = 0.f;
+  // a sink is a term of the denominator that was there first
+  float m = sinks != nullptr ? sinks[h] : -INFINITY, l = sinks != nullptr ? 1.f : 0.f;
   for (int u0 = 0; u0 < total; u0 += kWave) {
     const int u = u0 + lane;
     float s = -INFINITY;
@@ -428,7 +464,7 @@ __global__ __launch_bounds__(256, 2) void kv_attention_tile_kernel(
     const int* __restrict__ block_tables, int max_blocks, const int* __restrict__ query_start_loc,
     const int* __restrict__ context_lens, const float* __restrict__ out_inv_freq, int interleaved,
     int heads, int kv_heads, int block_size, int num_blocks, int window, float scale, int head_waves,
-    int keep_first, float softcap) {
+    int keep_first, float softcap, int chunk, const float* __restrict__ sinks) {
   using T = typename S::T;
   using M = Mfma16<S>;
   constexpr int D = 32 * DB, VD = 32 * VB;
@@ -459,7 +495,10 @@ __global__ __launch_bounds__(256, 2) void kv_attention_tile_kernel(
   const int p_first = context_lens[b] + tile_rows * tile_x, p_last = p_first + n_tile - 1;
   const int p0 = p_first + kTile * rb;                // this wave's first position
   const int pq = p0 + c;
-  const int j_lo = window > 0 ? max(0, p_first - window + 1) : 0;
+  const int j_lo = first_key(p_first, window, chunk);
+  const int lo_q = first_key(pq, window, chunk);      // this lane's row's first key
+  const int lo_first = first_key(p0, window, chunk);  // of the wave's first row and of its last
+  const int lo_last = first_key(p0 + kTile - 1, window, chunk);
   // the keys this workgroup walks, through one index: the kept first tokens that lie ahead of the
   // first row's window, then the window's first key to the last row
   const int nk = min(keep_first, j_lo);
@@ -483,6 +522,10 @@ __global__ __launch_bounds__(256, 2) void kv_attention_tile_kernel(
 #pragma unroll
     for (int i = 0; i < 16; ++i) o[n][i] = 0.f;
   float m = -INFINITY, l = 0.f;
+  if (sinks != nullptr && active) {       // the denominator's first term, counted in one lane half
+    m = sinks[h] * 1.4426950408889634f;
+    l = hf == 0 ? 1.f : 0.f;
+  }
 
   // threads 0 .. 63 look the rows of a tile up: the block id is read one step before it is used
   auto load_block = [&](int u0) {
@@ -560,7 +603,7 @@ __global__ __launch_bounds__(256, 2) void kv_attention_tile_kernel(
     const bool kept_tile = u0 < nk;
     const int j0 = u0 - nk + j_lo;            // the tile's first key when it holds window keys only
     if (active && (kept_tile || (j0 <= p0 + nq - 1 &&
-                                 !(window > 0 && j0 + kKeys - 1 < p0 - window + 1 && j0 >= keep_first)))) {
+                                 !(j0 + kKeys - 1 < lo_first && j0 >= keep_first)))) {
       f32x16 st[2];
 #pragma unroll
       for (int kb = 0; kb < 2; ++kb) {
@@ -573,8 +616,7 @@ __global__ __launch_bounds__(256, 2) void kv_attention_tile_kernel(
         }
       }
       // every key of the tile visible to every row of the wave: no masks
-      const bool full = !kept_tile && j0 + kKeys - 1 <= p0 && nq == kTile &&
-                        (window <= 0 || p0 + kTile - 1 - j0 < window);
+      const bool full = !kept_tile && j0 + kKeys - 1 <= p0 && nq == kTile && j0 >= lo_last;
       float mt = -INFINITY;
 #pragma unroll
       for (int kb = 0; kb < 2; ++kb)
@@ -584,8 +626,7 @@ __global__ __launch_bounds__(256, 2) void kv_attention_tile_kernel(
           if (softcap > 0.f) v = cap_score_fast(st[kb][i] * scale, cap2, cap_arg);
           if (!full) {
             const int j = key_of(u0 + 32 * kb + (i & 3) + 8 * (i >> 2) + 4 * hf);
-            const int dist = pq - j;
-            const bool ok = c < nq && dist >= 0 && (window <= 0 || dist < window || j < keep_first);
+            const bool ok = c < nq && j <= pq && (j >= lo_q || j < keep_first);
             v = ok ? v : -INFINITY;
           }
           st[kb][i] = v;
@@ -676,7 +717,7 @@ __global__ __launch_bounds__(64 * kRowWaves) void kv_attention_heads_kernel(
     const int* __restrict__ block_tables, int max_blocks, const int* __restrict__ token_seq,
     const int64_t* __restrict__ positions, const float* __restrict__ out_inv_freq, int interleaved,
     int heads, int kv_heads, int block_size, int num_blocks, int window, float scale,
-    int merge_heads, int keep_first, float softcap) {
+    int merge_heads, int keep_first, float softcap, int chunk, const float* __restrict__ sinks) {
   using T = typename S::T;
   using M = Mfma8<S>;
   constexpr int D = 32 * DB, VD = 32 * VB;
@@ -695,7 +736,7 @@ __global__ __launch_bounds__(64 * kRowWaves) void kv_attention_heads_kernel(
   const int nh = min(32, g * group + group - h0);
   const int p = (int)positions[t];
   const int* table = block_tables + (int64_t)token_seq[t] * max_blocks;
-  const int lo = window > 0 ? max(0, p - window + 1) : 0;
+  const int lo = first_key(p, window, chunk);
   const int nk = min(keep_first, lo);         // kept keys ahead of the window
   const int total = nk + p - lo + 1;
   const float cap_arg = softcap > 0.f ? 2.f * 1.4426950408889634f / softcap : 0.f;
@@ -714,6 +755,10 @@ __global__ __launch_bounds__(64 * kRowWaves) void kv_attention_heads_kernel(
 #pragma unroll
     for (int i = 0; i < 16; ++i) o[n][i] = 0.f;
   float m = -INFINITY, l = 0.f;
+  if (sinks != nullptr && live && w == 0) {   // the denominator's first term, counted by one wave's lane half
+    m = sinks[h0 + c];
+    l = hf == 0 ? 1.f : 0.f;
+  }
 
   // A wave's share of a tile is D / 8 + VD / 8 pieces of 8 bytes per lane, all issued before any
   // is used and one tile ahead.  Lanes 0..31 look the 32 tokens of the tile up once and hand the
@@ -869,7 +914,8 @@ int launch_heads_one(dim3 grid, hipStream_t stream, typename S::T* out, int64_t 
                      const typename S::T* value_cache, const int* block_tables, int max_blocks,
                      const int* token_seq, const int64_t* positions, const float* out_inv_freq,
                      int interleaved, int heads, int kv_heads, int block_size, int num_blocks,
-                     int window, float scale, int keep_first, float softcap) {
+                     int window, float scale, int keep_first, float softcap, int chunk,
+                     const float* sinks) {
   constexpr int D = 32 * DB, VD = 32 * VB;
   const int group = heads / kv_heads;
   const int merge_heads = group < 32 ? group : 32;
@@ -887,7 +933,7 @@ int launch_heads_one(dim3 grid, hipStream_t stream, typename S::T* out, int64_t 
   kv_attention_heads_kernel<S, DB, VB><<<grid, 64 * kRowWaves, lds, stream>>>(
       out, out_stride, q, q_stride, gate, gate_stride, key_cache, value_cache, block_tables,
       max_blocks, token_seq, positions, out_inv_freq, interleaved, heads, kv_heads, block_size,
-      num_blocks, window, scale, merge_heads, keep_first, softcap);
+      num_blocks, window, scale, merge_heads, keep_first, softcap, chunk, sinks);
   VLA_SEQ_HIP_CHECK(hipGetLastError());
   return VLA_OK;
 }
@@ -899,11 +945,12 @@ int launch_tiles_one(dim3 grid, hipStream_t stream, typename S::T* out, int64_t 
                      const typename S::T* value_cache, const int* block_tables, int max_blocks,
                      const int* qsl, const int* ctx, const float* out_inv_freq, int interleaved,
                      int heads, int kv_heads, int block_size, int num_blocks, int window,
-                     float scale, int head_waves, int keep_first, float softcap) {
+                     float scale, int head_waves, int keep_first, float softcap, int chunk,
+                     const float* sinks) {
   kv_attention_tile_kernel<S, DB, VB><<<grid, 256, 0, stream>>>(
       out, out_stride, q, q_stride, gate, gate_stride, key_cache, value_cache, block_tables,
       max_blocks, qsl, ctx, out_inv_freq, interleaved, heads, kv_heads, block_size, num_blocks,
-      window, scale, head_waves, keep_first, softcap);
+      window, scale, head_waves, keep_first, softcap, chunk, sinks);
   VLA_SEQ_HIP_CHECK(hipGetLastError());
   return VLA_OK;
 }
@@ -959,7 +1006,7 @@ extern "C" int vla_seq_rotary_kv_write(void* q, int64_t q_stride, const void* k,
                                        int interleaved, int block_size, int num_blocks, int dtype,
                                        const float* q_norm, const float* k_norm, float norm_eps,
                                        const void* v_other, int64_t v_other_stride,
-                                       const float* v_blend, void* stream) {
+                                       const float* v_blend, int head_norm, void* stream) {
   if (num_tokens == 0) return VLA_OK;
   if (!q || !k || !v || !key_cache || !value_cache || !positions || !slot_mapping || num_tokens < 0 ||
       heads <= 0 || kv_heads <= 0 || dim <= 0 || vdim <= 0 || rot_dims < 0 || rot_dims > dim ||
@@ -971,11 +1018,12 @@ extern "C" int vla_seq_rotary_kv_write(void* q, int64_t q_stride, const void* k,
   return with_dtype(dtype, [&](auto s) {
     using S = decltype(s);
     using T = typename S::T;
-    rotary_kv_write_kernel<S><<<num_tokens, 256, 0, (hipStream_t)stream>>>(
+    const size_t lds = head_norm ? sizeof(float) * ((size_t)heads + kv_heads) : 0;
+    rotary_kv_write_kernel<S><<<num_tokens, 256, lds, (hipStream_t)stream>>>(
         (T*)q, q_stride, (const T*)k, k_stride, (const T*)v, v_stride, (T*)key_cache,
         (T*)value_cache, positions, slot_mapping, inv_freq, value_inv_freq, heads, kv_heads, dim,
         vdim, rot_dims, interleaved, (int64_t)num_blocks * block_size, q_norm, k_norm, norm_eps,
-        (const T*)v_other, v_other_stride, v_blend);
+        (const T*)v_other, v_other_stride, v_blend, head_norm);
     VLA_SEQ_HIP_CHECK(hipGetLastError());
     return VLA_OK;
   });
@@ -988,7 +1036,8 @@ extern "C" int vla_seq_kv_attention(void* out, int64_t out_stride, const void* q
                                     const float* out_inv_freq, int interleaved, int num_tokens,
                                     int heads, int kv_heads, int dim, int vdim, int block_size,
                                     int num_blocks, int window, float scale, int dtype,
-                                    int keep_first, float softcap, void* stream) {
+                                    int keep_first, float softcap, int chunk, const float* sinks,
+                                    void* stream) {
   if (num_tokens == 0) return VLA_OK;
   if (!out || !q || !key_cache || !value_cache || !block_tables || !token_seq || !positions ||
       num_tokens < 0 || heads <= 0 || kv_heads <= 0 || heads % kv_heads != 0 || block_size <= 0 ||
@@ -996,6 +1045,7 @@ extern "C" int vla_seq_kv_attention(void* out, int64_t out_stride, const void* q
       q_stride < (int64_t)heads * dim || (gate && gate_stride < heads) || keep_first < 0 ||
       !(softcap >= 0.f))
     return VLA_ERR_ARG;
+  if (window <= 0 && chunk <= 0) keep_first = 0;
   if (dim <= 0 || dim > kMaxDim || vdim <= 0 || vdim > kMaxDim) return VLA_ERR_HEAD_SIZE;
   return with_dtype(dtype, [&](auto s) {
     using S = decltype(s);
@@ -1012,7 +1062,7 @@ extern "C" int vla_seq_kv_attention(void* out, int64_t out_stride, const void* q
                                        (const T*)key_cache, (const T*)value_cache, block_tables,
                                        max_blocks, token_seq, positions, out_inv_freq, interleaved,
                                        heads, kv_heads, block_size, num_blocks, window, scale,
-                                       window > 0 ? keep_first : 0, softcap);
+                                       keep_first, softcap, chunk, sinks);
         if (rc != VLA_ERR_HEAD_SIZE) return rc;
       }
     }
@@ -1021,7 +1071,7 @@ extern "C" int vla_seq_kv_attention(void* out, int64_t out_stride, const void* q
         (T*)out, out_stride, (const T*)q, q_stride, (const T*)gate, gate_stride,
         (const T*)key_cache, (const T*)value_cache, block_tables, max_blocks, token_seq, positions,
         out_inv_freq, interleaved, heads, kv_heads, dim, vdim, block_size, num_blocks, window, scale,
-        window > 0 ? keep_first : 0, softcap);
+        keep_first, softcap, chunk, sinks);
     VLA_SEQ_HIP_CHECK(hipGetLastError());
     return VLA_OK;
   });
@@ -1045,10 +1095,10 @@ extern "C" int vla_seq_kv_attention_tiles(
     int max_blocks, const int* query_start_loc, const int* context_lens, const float* out_inv_freq,
     int interleaved, int num_seqs, int max_query_len, int heads, int kv_heads, int dim, int vdim,
     int block_size, int num_blocks, int window, float scale, int dtype, int keep_first,
-    float softcap, void* stream) {
+    float softcap, int chunk, const float* sinks, void* stream) {
   if (num_seqs == 0 || max_query_len == 0) return VLA_OK;
   if (keep_first < 0 || !(softcap >= 0.f)) return VLA_ERR_ARG;
-  if (window <= 0) keep_first = 0;
+  if (window <= 0 && chunk <= 0) keep_first = 0;
   if (!out || !q || !key_cache || !value_cache || !block_tables || !query_start_loc || !context_lens ||
       num_seqs < 0 || num_seqs > 65535 || max_query_len < 0 || heads <= 0 || kv_heads <= 0 ||
       heads % kv_heads != 0 || block_size <= 0 || num_blocks <= 0 || max_blocks <= 0 ||
@@ -1075,11 +1125,11 @@ extern "C" int vla_seq_kv_attention_tiles(
                               (const __bf16*)key_cache, (const __bf16*)value_cache, block_tables,
                               max_blocks, query_start_loc, context_lens, out_inv_freq, interleaved,
                               heads, kv_heads, block_size, num_blocks, window, scale, head_waves,
-                              keep_first, softcap);
+                              keep_first, softcap, chunk, sinks);
   return launch_tiles<F16>(dim / 32, vdim / 32, grid, (hipStream_t)stream, (_Float16*)out, out_stride,
                            (const _Float16*)q, q_stride, (const _Float16*)gate, gate_stride,
                            (const _Float16*)key_cache, (const _Float16*)value_cache, block_tables,
                            max_blocks, query_start_loc, context_lens, out_inv_freq, interleaved, heads,
                            kv_heads, block_size, num_blocks, window, scale, head_waves, keep_first,
-                           softcap);
+                           softcap, chunk, sinks);
 }

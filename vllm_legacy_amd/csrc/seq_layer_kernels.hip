@@ -13,17 +13,19 @@ constexpr int kThreads = 256;
 constexpr int kKeep = 8;          // row elements a thread keeps in registers (rows up to 2048)
 constexpr int kMaxTaps = 32;
 
-template <class SY, class SO>
+// TWO: a second branch y2 is normed by itself and added beside the first (parallel mixers).
+template <class SY, class SO, bool TWO>
 __global__ __launch_bounds__(kThreads) void residual_norms_kernel(
     float* __restrict__ x, const typename SY::T* __restrict__ y, int64_t y_stride,
     const float* __restrict__ y_bias, const float* __restrict__ post_w,
     const float* __restrict__ layer_scale,
     const float* __restrict__ add_row, typename SO::T* __restrict__ out,
-    const float* __restrict__ pre_w, float eps, int width) {
+    const float* __restrict__ pre_w, float eps, int width, float y_scale,
+    const typename SY::T* __restrict__ y2, int64_t y2_stride, const float* __restrict__ post_w2) {
   __shared__ float red[16];
   const int64_t base = (int64_t)blockIdx.x * width;
-  float keep[kKeep], keepx[kKeep];
-  float inv_y = 0.f;
+  float keep[kKeep], keepx[kKeep], keep2[TWO ? kKeep : 1];
+  float inv_y = 1.f, inv_y2 = 1.f;
   // the stream's row is asked for before the first reduction, so its latency hides behind it
 #pragma unroll
   for (int i = 0; i < kKeep; ++i) {
@@ -32,30 +34,46 @@ __global__ __launch_bounds__(kThreads) void residual_norms_kernel(
   }
   if (y != nullptr) {
     const typename SY::T* yr = y + (int64_t)blockIdx.x * y_stride;
-    float ss = 0.f;
+    const typename SY::T* yr2 = TWO ? y2 + (int64_t)blockIdx.x * y2_stride : nullptr;
+    float ss = 0.f, ss2 = 0.f;
 #pragma unroll
     for (int i = 0; i < kKeep; ++i) {
       const int c = threadIdx.x + i * kThreads;
       if (c < width) {
         keep[i] = SY::to_f32(yr[c]) + (y_bias != nullptr ? y_bias[c] : 0.f);
         ss += keep[i] * keep[i];
+        if constexpr (TWO) {
+          keep2[i] = SY::to_f32(yr2[c]);
+          ss2 += keep2[i] * keep2[i];
+        }
       }
     }
-    for (int c = threadIdx.x + kKeep * kThreads; c < width; c += kThreads) {
-      const float v = SY::to_f32(yr[c]) + (y_bias != nullptr ? y_bias[c] : 0.f);
-      ss += v * v;
+    if (post_w != nullptr) {
+      for (int c = threadIdx.x + kKeep * kThreads; c < width; c += kThreads) {
+        const float v = SY::to_f32(yr[c]) + (y_bias != nullptr ? y_bias[c] : 0.f);
+        ss += v * v;
+        if constexpr (TWO) {
+          const float v2 = SY::to_f32(yr2[c]);
+          ss2 += v2 * v2;
+        }
+      }
+      ss = block_sum(ss, red);
+      inv_y = 1.f / sqrtf(ss / (float)width + eps);
+      if constexpr (TWO) {
+        ss2 = block_sum(ss2, red);
+        inv_y2 = 1.f / sqrtf(ss2 / (float)width + eps);
+      }
     }
-    ss = block_sum(ss, red);
-    inv_y = 1.f / sqrtf(ss / (float)width + eps);
   }
   const bool writes = y != nullptr || add_row != nullptr;
   float ss = 0.f;
-  auto update = [&](int c, float xv, float yv) {
+  auto update = [&](int c, float xv, float yv, float yv2) {
     float v = xv;
     if (y != nullptr) {
-      float u = yv * inv_y * post_w[c];
+      float u = post_w != nullptr ? yv * inv_y * post_w[c] : yv;
       if (layer_scale != nullptr) u *= layer_scale[c];
-      v += u;
+      if constexpr (TWO) u += yv2 * inv_y2 * post_w2[c];
+      v += u * y_scale;
     }
     if (add_row != nullptr) v += add_row[c];
     if (writes) x[base + c] = v;
@@ -65,12 +83,15 @@ __global__ __launch_bounds__(kThreads) void residual_norms_kernel(
 #pragma unroll
   for (int i = 0; i < kKeep; ++i) {
     const int c = threadIdx.x + i * kThreads;
-    if (c < width) keep[i] = update(c, keepx[i], y != nullptr ? keep[i] : 0.f);
+    if (c < width) keep[i] = update(c, keepx[i], y != nullptr ? keep[i] : 0.f, TWO ? keep2[TWO ? i : 0] : 0.f);
   }
-  for (int c = threadIdx.x + kKeep * kThreads; c < width; c += kThreads)
-    update(c, x[base + c], y != nullptr ? SY::to_f32(y[(int64_t)blockIdx.x * y_stride + c]) +
-                                              (y_bias != nullptr ? y_bias[c] : 0.f)
-                                        : 0.f);
+  for (int c = threadIdx.x + kKeep * kThreads; c < width; c += kThreads) {
+    float yv = 0.f, yv2 = 0.f;
+    if (y != nullptr)
+      yv = SY::to_f32(y[(int64_t)blockIdx.x * y_stride + c]) + (y_bias != nullptr ? y_bias[c] : 0.f);
+    if constexpr (TWO) yv2 = SY::to_f32(y2[(int64_t)blockIdx.x * y2_stride + c]);
+    update(c, x[base + c], yv, yv2);
+  }
   if (out == nullptr) return;
   if (pre_w == nullptr) {           // no norm ahead of the reader: the stream's row as it is
 #pragma unroll
@@ -226,16 +247,24 @@ extern "C" int vla_seq_residual_norms(float* x, const void* y, int64_t y_stride,
                                       const float* layer_scale,
                                       const float* add_row, void* out, const float* pre_weight,
                                       float eps, int num_tokens, int width, int out_dtype,
-                                      void* stream) {
+                                      float y_scale, const void* y2, int64_t y2_stride,
+                                      const float* post_weight2, void* stream) {
   if (num_tokens == 0) return VLA_OK;
-  if (!x || num_tokens < 0 || width <= 0 || (y && (!post_weight || y_stride < width)))
+  if (!x || num_tokens < 0 || width <= 0 || (y && y_stride < width) ||
+      (y2 && (!y || !post_weight || !post_weight2 || y2_stride < width)))
     return VLA_ERR_ARG;
   return with_two_dtypes(y ? y_dtype : VLA_F32, out ? out_dtype : VLA_F32, [&](auto sy, auto so) {
     using SY = decltype(sy);
     using SO = decltype(so);
-    residual_norms_kernel<SY, SO><<<num_tokens, kThreads, 0, (hipStream_t)stream>>>(
-        x, (const typename SY::T*)y, y_stride, y_bias, post_weight, layer_scale, add_row,
-        (typename SO::T*)out, pre_weight, eps, width);
+    using TY = typename SY::T;
+    if (y2 != nullptr)
+      residual_norms_kernel<SY, SO, true><<<num_tokens, kThreads, 0, (hipStream_t)stream>>>(
+          x, (const TY*)y, y_stride, y_bias, post_weight, layer_scale, add_row, (typename SO::T*)out,
+          pre_weight, eps, width, y_scale, (const TY*)y2, y2_stride, post_weight2);
+    else
+      residual_norms_kernel<SY, SO, false><<<num_tokens, kThreads, 0, (hipStream_t)stream>>>(
+          x, (const TY*)y, y_stride, y_bias, post_weight, layer_scale, add_row, (typename SO::T*)out,
+          pre_weight, eps, width, y_scale, nullptr, 0, nullptr);
     VLA_SEQ_HIP_CHECK(hipGetLastError());
     return VLA_OK;
   });

@@ -1,11 +1,11 @@
 // Mixture-of-experts feed-forward in the activation dtype (no quantization), routed on the device
 // without a host synchronisation:
-//   moe_route      per token: router logits in fp32 (plus a bias), softmax over all experts, choice by score plus
-//                  a per-expert correction, weights = chosen scores renormalized; also the sigmoid
-//                  gate of a shared expert
+//   moe_route      per token: router logits in fp32 (plus a bias), softmax over all experts or the
+//                  sigmoid of each logit, choice by score plus a per-expert correction, weights = chosen
+//                  scores, renormalized or as they are; also the sigmoid gate of a shared expert
 //   moe_plan       groups the (token, choice) pairs by expert into row tiles of kTile rows (groups
 //                  are padded to whole tiles, so a tile belongs to one expert)
-//   grouped_linear out[row] = act(W_e a[row]) for the rows of every tile, W_e the tile's expert;
+//   grouped_linear out[row] = act(W_e a[row] * scale[row]) for the rows of every tile, W_e the tile's expert;
 //                  the rows of the first product are gathered from the tokens on the fly
 //   moe_combine    per token: weighted sum of its experts' rows (a choice without a row is an
 //                  identity expert: the token's own input), plus the gated shared expert
@@ -43,7 +43,7 @@ __global__ __launch_bounds__(256) void moe_route_kernel(
     const float* __restrict__ logits, int64_t logits_stride, const float* __restrict__ bias,
     const float* __restrict__ correction,
     const float* __restrict__ shared_gate_w, int* __restrict__ experts, float* __restrict__ weights,
-    float* __restrict__ shared_gate, int width, int routed, int top) {
+    float* __restrict__ shared_gate, int width, int routed, int top, int score, int renormalize) {
   __shared__ float z[kMaxRouted + 1];
   const int t = blockIdx.x, lane = threadIdx.x & 63, w = threadIdx.x >> 6;
   const bool gated = shared_gate != nullptr;
@@ -66,25 +66,34 @@ __global__ __launch_bounds__(256) void moe_route_kernel(
   if (gated && lane == 0) shared_gate[t] = 1.f / (1.f + expf(-z[routed]));
   constexpr int PER = kMaxRouted / kWave;
   float s[PER], choice[PER];
-  float mx = -INFINITY;
+  if (score == VLA_SCORE_SIGMOID) {
+#pragma unroll
+    for (int i = 0; i < PER; ++i) {
+      const int n = lane + i * kWave;
+      s[i] = n < routed ? 1.f / (1.f + expf(-z[n])) : 0.f;
+    }
+  } else {
+    float mx = -INFINITY;
+#pragma unroll
+    for (int i = 0; i < PER; ++i) {
+      const int n = lane + i * kWave;
+      s[i] = n < routed ? z[n] : -INFINITY;
+      mx = fmaxf(mx, s[i]);
+    }
+    mx = wave_max(mx);
+    float sum = 0.f;
+#pragma unroll
+    for (int i = 0; i < PER; ++i) {
+      s[i] = lane + i * kWave < routed ? expf(s[i] - mx) : 0.f;
+      sum += s[i];
+    }
+    sum = wave_sum(sum);
+#pragma unroll
+    for (int i = 0; i < PER; ++i) s[i] /= sum;
+  }
 #pragma unroll
   for (int i = 0; i < PER; ++i) {
     const int n = lane + i * kWave;
-    s[i] = n < routed ? z[n] : -INFINITY;
-    mx = fmaxf(mx, s[i]);
-  }
-  mx = wave_max(mx);
-  float sum = 0.f;
-#pragma unroll
-  for (int i = 0; i < PER; ++i) {
-    s[i] = lane + i * kWave < routed ? expf(s[i] - mx) : 0.f;
-    sum += s[i];
-  }
-  sum = wave_sum(sum);
-#pragma unroll
-  for (int i = 0; i < PER; ++i) {
-    const int n = lane + i * kWave;
-    s[i] /= sum;
     choice[i] = n < routed ? s[i] + (correction != nullptr ? correction[n] : 0.f) : -INFINITY;
   }
   float total = 0.f, mine = 0.f;     // lane k keeps the k-th chosen score
@@ -122,7 +131,7 @@ __global__ __launch_bounds__(256) void moe_route_kernel(
   }
   if (lane < top) {
     experts[(int64_t)t * top + lane] = mine_e;
-    weights[(int64_t)t * top + lane] = mine / (total + 1e-20f);
+    weights[(int64_t)t * top + lane] = renormalize ? mine / (total + 1e-20f) : mine;
   }
 }
 
@@ -131,7 +140,7 @@ __global__ __launch_bounds__(256) void moe_route_kernel(
 __global__ __launch_bounds__(1024) void moe_plan_kernel(
     const int* __restrict__ experts, int num_pairs, int top, int num_experts,
     int* __restrict__ pair_row, int* __restrict__ row_token, int* __restrict__ tile_expert,
-    int max_tiles) {
+    int max_tiles, const float* __restrict__ weights, float* __restrict__ row_weight) {
   extern __shared__ int lds[];
   int* count = lds;                      // [num_experts]
   int* offset = lds + num_experts;       // [num_experts + 1], in rows
@@ -162,10 +171,12 @@ __global__ __launch_bounds__(1024) void moe_plan_kernel(
     int row = -1;
     if (e >= 0 && e < num_experts) {
       row = offset[e] + atomicAdd(&cursor[e], 1);
-      if (row < max_tiles * kTile)
+      if (row < max_tiles * kTile) {
         row_token[row] = i / top;
-      else
+        if (row_weight != nullptr) row_weight[row] = weights[i];
+      } else {
         row = -1;
+      }
     }
     pair_row[i] = row;
   }
@@ -199,7 +210,8 @@ template <class S, class SO>
 __global__ __launch_bounds__(256) void grouped_linear_mfma_kernel(
     typename SO::T* __restrict__ out, int64_t out_stride, const typename S::T* __restrict__ a,
     int64_t a_stride, const int* __restrict__ row_token, const typename S::T* __restrict__ weight,
-    const int* __restrict__ tile_expert, int n_out, int k_in, int act) {
+    const int* __restrict__ tile_expert, int n_out, int k_in, int act,
+    const float* __restrict__ row_scale) {
   using T = typename S::T;
   const int tile = blockIdx.x;
   const int e = tile_expert[tile];
@@ -221,10 +233,11 @@ __global__ __launch_bounds__(256) void grouped_linear_mfma_kernel(
     const u32x2 wv = *reinterpret_cast<const u32x2*>(wr + k);
     acc = Mma<S>::run(wv, av, acc);
   }
+  const float sc = row_scale != nullptr && src >= 0 ? row_scale[row] : 1.f;
 #pragma unroll
   for (int i = 0; i < 16; ++i) {
     const int n = n0 + (i & 3) + 8 * (i >> 2) + 4 * hf;
-    if (n < n_out) out[(int64_t)row * out_stride + n] = SO::from_f32(act_apply(acc[i], act));
+    if (n < n_out) out[(int64_t)row * out_stride + n] = SO::from_f32(act_apply(acc[i] * sc, act));
   }
 }
 
@@ -256,7 +269,8 @@ __device__ __forceinline__ void grouped_run(typename SO::T* __restrict__ out, in
                                             const typename S::T* __restrict__ a, int64_t a_stride,
                                             const int* __restrict__ row_token,
                                             const typename S::T* __restrict__ wr, int first_tile, int n0,
-                                            int n_out, int k_in, int act, int hf, int c) {
+                                            int n_out, int k_in, int act,
+                                            const float* __restrict__ row_scale, int hf, int c) {
   using T = typename S::T;
   const T* ar[C];
   bool live[C];
@@ -283,10 +297,12 @@ __device__ __forceinline__ void grouped_run(typename SO::T* __restrict__ out, in
 #pragma unroll
   for (int r = 0; r < C; ++r) {
     const int row = (first_tile + r) * kTile + c;
+    // a padding row's sums are zeros and its scale was never written
+    const float sc = row_scale != nullptr && (row_token == nullptr || row_token[row] >= 0) ? row_scale[row] : 1.f;
 #pragma unroll
     for (int i = 0; i < 16; ++i) {
       const int n = n0 + (i & 3) + 8 * (i >> 2) + 4 * hf;
-      if (n < n_out) out[(int64_t)row * out_stride + n] = SO::from_f32(act_apply(acc[r][i], act));
+      if (n < n_out) out[(int64_t)row * out_stride + n] = SO::from_f32(act_apply(acc[r][i] * sc, act));
     }
   }
 }
@@ -296,7 +312,7 @@ __global__ __launch_bounds__(256) void grouped_linear_mfma16_kernel(
     typename SO::T* __restrict__ out, int64_t out_stride, const typename S::T* __restrict__ a,
     int64_t a_stride, const int* __restrict__ row_token, const typename S::T* __restrict__ weight,
     const int* __restrict__ tile_expert, int max_tiles, int n_out, int k_in, int act,
-    int tiles_per_group) {
+    const float* __restrict__ row_scale, int tiles_per_group) {
   const int lane = threadIdx.x & 63, w = threadIdx.x >> 6;
   const int hf = lane >> 5, c = lane & 31;
   const int n0 = (blockIdx.y * (blockDim.x >> 6) + w) * 32;
@@ -314,10 +330,10 @@ __global__ __launch_bounds__(256) void grouped_linear_mfma16_kernel(
     while (j < last && tile_expert[j] == e) ++j;
     const typename S::T* wr = weight + ((int64_t)e * n_out + min(n0 + c, n_out - 1)) * k_in + 8 * hf;
     switch (j - i) {
-      case 1: grouped_run<S, SO, 1>(out, out_stride, a, a_stride, row_token, wr, i, n0, n_out, k_in, act, hf, c); break;
-      case 2: grouped_run<S, SO, 2>(out, out_stride, a, a_stride, row_token, wr, i, n0, n_out, k_in, act, hf, c); break;
-      case 3: grouped_run<S, SO, 3>(out, out_stride, a, a_stride, row_token, wr, i, n0, n_out, k_in, act, hf, c); break;
-      default: grouped_run<S, SO, 4>(out, out_stride, a, a_stride, row_token, wr, i, n0, n_out, k_in, act, hf, c); break;
+      case 1: grouped_run<S, SO, 1>(out, out_stride, a, a_stride, row_token, wr, i, n0, n_out, k_in, act, row_scale, hf, c); break;
+      case 2: grouped_run<S, SO, 2>(out, out_stride, a, a_stride, row_token, wr, i, n0, n_out, k_in, act, row_scale, hf, c); break;
+      case 3: grouped_run<S, SO, 3>(out, out_stride, a, a_stride, row_token, wr, i, n0, n_out, k_in, act, row_scale, hf, c); break;
+      default: grouped_run<S, SO, 4>(out, out_stride, a, a_stride, row_token, wr, i, n0, n_out, k_in, act, row_scale, hf, c); break;
     }
     i = j;
   }
@@ -337,7 +353,8 @@ __device__ __forceinline__ void grouped_run_lds(typename S::T* __restrict__ a_ld
                                                 const typename S::T* __restrict__ a, int64_t a_stride,
                                                 const int* __restrict__ row_token,
                                                 const typename S::T* __restrict__ wr, int first_tile, int n0,
-                                                int n_out, int k_in, int act, int hf, int c) {
+                                                int n_out, int k_in, int act,
+                                            const float* __restrict__ row_scale, int hf, int c) {
   using T = typename S::T;
   const int tid = threadIdx.x;
   // staging: C pieces of 16 bytes per thread and chunk; piece p = tid + 256 u is row p / 8, values 8 (p % 8) ..
@@ -392,10 +409,12 @@ __device__ __forceinline__ void grouped_run_lds(typename S::T* __restrict__ a_ld
 #pragma unroll
   for (int r = 0; r < C; ++r) {
     const int row = (first_tile + r) * kTile + c;
+    // a padding row's sums are zeros and its scale was never written
+    const float sc = row_scale != nullptr && (row_token == nullptr || row_token[row] >= 0) ? row_scale[row] : 1.f;
 #pragma unroll
     for (int i = 0; i < 16; ++i) {
       const int n = n0 + (i & 3) + 8 * (i >> 2) + 4 * hf;
-      if (n < n_out) out[(int64_t)row * out_stride + n] = SO::from_f32(act_apply(acc[r][i], act));
+      if (n < n_out) out[(int64_t)row * out_stride + n] = SO::from_f32(act_apply(acc[r][i] * sc, act));
     }
   }
 }
@@ -404,7 +423,8 @@ template <class S, class SO>
 __global__ __launch_bounds__(256) void grouped_linear_lds_kernel(
     typename SO::T* __restrict__ out, int64_t out_stride, const typename S::T* __restrict__ a,
     int64_t a_stride, const int* __restrict__ row_token, const typename S::T* __restrict__ weight,
-    const int* __restrict__ tile_expert, int max_tiles, int n_out, int k_in, int act) {
+    const int* __restrict__ tile_expert, int max_tiles, int n_out, int k_in, int act,
+    const float* __restrict__ row_scale) {
   __shared__ __align__(16) typename S::T a_lds[2 * 4 * kTile * kARow];
   const int lane = threadIdx.x & 63, w = threadIdx.x >> 6;
   const int hf = lane >> 5, c = lane & 31;
@@ -422,10 +442,10 @@ __global__ __launch_bounds__(256) void grouped_linear_lds_kernel(
     while (j < last && tile_expert[j] == e) ++j;
     const typename S::T* wr = weight + ((int64_t)e * n_out + min(n0 + c, n_out - 1)) * k_in + 8 * hf;
     switch (j - i) {
-      case 1: grouped_run_lds<S, SO, 1>(a_lds, out, out_stride, a, a_stride, row_token, wr, i, n0, n_out, k_in, act, hf, c); break;
-      case 2: grouped_run_lds<S, SO, 2>(a_lds, out, out_stride, a, a_stride, row_token, wr, i, n0, n_out, k_in, act, hf, c); break;
-      case 3: grouped_run_lds<S, SO, 3>(a_lds, out, out_stride, a, a_stride, row_token, wr, i, n0, n_out, k_in, act, hf, c); break;
-      default: grouped_run_lds<S, SO, 4>(a_lds, out, out_stride, a, a_stride, row_token, wr, i, n0, n_out, k_in, act, hf, c); break;
+      case 1: grouped_run_lds<S, SO, 1>(a_lds, out, out_stride, a, a_stride, row_token, wr, i, n0, n_out, k_in, act, row_scale, hf, c); break;
+      case 2: grouped_run_lds<S, SO, 2>(a_lds, out, out_stride, a, a_stride, row_token, wr, i, n0, n_out, k_in, act, row_scale, hf, c); break;
+      case 3: grouped_run_lds<S, SO, 3>(a_lds, out, out_stride, a, a_stride, row_token, wr, i, n0, n_out, k_in, act, row_scale, hf, c); break;
+      default: grouped_run_lds<S, SO, 4>(a_lds, out, out_stride, a, a_stride, row_token, wr, i, n0, n_out, k_in, act, row_scale, hf, c); break;
     }
     i = j;
   }
@@ -437,7 +457,8 @@ template <class S, class SO>
 __global__ __launch_bounds__(256) void grouped_linear_kernel(
     typename SO::T* __restrict__ out, int64_t out_stride, const typename S::T* __restrict__ a,
     int64_t a_stride, const int* __restrict__ row_token, const typename S::T* __restrict__ weight,
-    const int* __restrict__ tile_expert, int n_out, int k_in, int act) {
+    const int* __restrict__ tile_expert, int n_out, int k_in, int act,
+    const float* __restrict__ row_scale) {
   using T = typename S::T;
   const int tile = blockIdx.x;
   const int e = tile_expert[tile];
@@ -465,7 +486,8 @@ __global__ __launch_bounds__(256) void grouped_linear_kernel(
 #pragma unroll
   for (int r = 0; r < 8; ++r) {
     const int row = tile * kTile + w * 8 + r;
-    out[(int64_t)row * out_stride + n] = SO::from_f32(act_apply(live[r] ? acc[r] : 0.f, act));
+    const float sc = row_scale != nullptr && live[r] ? row_scale[row] : 1.f;
+    out[(int64_t)row * out_stride + n] = SO::from_f32(act_apply(live[r] ? acc[r] * sc : 0.f, act));
   }
 }
 
@@ -480,7 +502,7 @@ __global__ __launch_bounds__(256) void moe_combine_kernel(
     for (int k = 0; k < top; ++k) {
       const int row = pair_row[t * top + k];
       const float v = row >= 0 ? y[(int64_t)row * width + c] : S::to_f32(h[t * h_stride + c]);
-      acc += weights[t * top + k] * v;
+      acc += (weights != nullptr ? weights[t * top + k] : 1.f) * v;
     }
     if (shared_y != nullptr)
       acc += (shared_gate != nullptr ? shared_gate[t] : 1.f) * shared_y[t * width + c];
@@ -504,11 +526,13 @@ extern "C" int vla_seq_moe_route(const void* h, int64_t h_stride, const float* r
                                  const float* logits, int64_t logits_stride, const float* bias,
                                  const float* correction, const float* shared_gate_weight,
                                  int* experts, float* weights, float* shared_gate, int num_tokens,
-                                 int width, int routed, int top, int dtype, void* stream) {
+                                 int width, int routed, int top, int score, int renormalize, int dtype,
+                                 void* stream) {
   if (num_tokens == 0) return VLA_OK;
   const bool gated = shared_gate != nullptr;
   if (!experts || !weights || num_tokens < 0 || width <= 0 || routed <= 0 || routed > kMaxRouted ||
       top <= 0 || top > routed || top > kWave ||
+      (score != VLA_SCORE_SOFTMAX && score != VLA_SCORE_SIGMOID) ||
       (logits ? logits_stride < routed + (gated ? 1 : 0)
               : (!h || !router || h_stride < width || (gated && !shared_gate_weight))))
     return VLA_ERR_ARG;
@@ -516,7 +540,7 @@ extern "C" int vla_seq_moe_route(const void* h, int64_t h_stride, const float* r
     using S = decltype(s);
     moe_route_kernel<S><<<num_tokens, 256, 0, (hipStream_t)stream>>>(
         (const typename S::T*)h, h_stride, router, logits, logits_stride, bias, correction,
-        shared_gate_weight, experts, weights, shared_gate, width, routed, top);
+        shared_gate_weight, experts, weights, shared_gate, width, routed, top, score, renormalize);
     VLA_SEQ_HIP_CHECK(hipGetLastError());
     return VLA_OK;
   });
@@ -526,13 +550,14 @@ extern "C" int vla_seq_moe_tile_rows(void) { return kTile; }
 
 extern "C" int vla_seq_moe_plan(const int* experts, int num_tokens, int top, int num_experts,
                                 int* pair_row, int* row_token, int* tile_expert, int max_tiles,
-                                void* stream) {
-  if (!experts || !pair_row || !row_token || !tile_expert || num_tokens < 0 || top <= 0 ||
+                                const float* weights, float* row_weight, void* stream) {
+  if ((row_weight && !weights) || !experts || !pair_row || !row_token || !tile_expert || num_tokens < 0 || top <= 0 ||
       num_experts <= 0 || num_experts > 4096 || max_tiles <= 0)
     return VLA_ERR_ARG;
   const size_t lds = sizeof(int) * (3 * (size_t)num_experts + 1);
   moe_plan_kernel<<<1, 1024, lds, (hipStream_t)stream>>>(experts, num_tokens * top, top, num_experts,
-                                                        pair_row, row_token, tile_expert, max_tiles);
+                                                        pair_row, row_token, tile_expert, max_tiles,
+                                                        weights, row_weight);
   VLA_SEQ_HIP_CHECK(hipGetLastError());
   return VLA_OK;
 }
@@ -540,7 +565,7 @@ extern "C" int vla_seq_moe_plan(const int* experts, int num_tokens, int top, int
 extern "C" int vla_seq_grouped_linear(void* out, int64_t out_stride, int out_dtype, const void* a,
                                       int64_t a_stride, const int* row_token, const void* weight,
                                       const int* tile_expert, int max_tiles, int n_out, int k_in,
-                                      int act, int dtype, void* stream) {
+                                      int act, const float* row_scale, int dtype, void* stream) {
   if (max_tiles == 0) return VLA_OK;
   if (!out || !a || !weight || !tile_expert || max_tiles < 0 || n_out <= 0 || k_in <= 0 ||
       out_stride < n_out || a_stride < k_in || act < VLA_ACT_NONE || act > VLA_ACT_GELU_TANH)
@@ -561,7 +586,7 @@ extern "C" int vla_seq_grouped_linear(void* out, int64_t out_stride, int out_dty
           grouped_linear_lds_kernel<S, SO>
               <<<dim3((max_tiles + kRunTiles - 1) / kRunTiles, (n_out + 127) / 128), 256, 0, st>>>(
                   (typename SO::T*)out, out_stride, (const T*)a, a_stride, row_token, (const T*)weight,
-                  tile_expert, max_tiles, n_out, k_in, act);
+                  tile_expert, max_tiles, n_out, k_in, act, row_scale);
           VLA_SEQ_HIP_CHECK(hipGetLastError());
           return VLA_OK;
         }
@@ -569,21 +594,21 @@ extern "C" int vla_seq_grouped_linear(void* out, int64_t out_stride, int out_dty
         grouped_linear_mfma16_kernel<S, SO>
             <<<dim3((max_tiles + per - 1) / per, (n_out + 32 * waves - 1) / (32 * waves)), 64 * waves, 0, st>>>(
                 (typename SO::T*)out, out_stride, (const T*)a, a_stride, row_token, (const T*)weight,
-                tile_expert, max_tiles, n_out, k_in, act, per);
+                tile_expert, max_tiles, n_out, k_in, act, row_scale, per);
         VLA_SEQ_HIP_CHECK(hipGetLastError());
         return VLA_OK;
       }
       if (k_in % 8 == 0 && ((uintptr_t)a % 8) == 0 && (a_stride % 4) == 0 && ((uintptr_t)weight % 8) == 0) {
         grouped_linear_mfma_kernel<S, SO><<<dim3(max_tiles, (n_out + 127) / 128), 256, 0, st>>>(
             (typename SO::T*)out, out_stride, (const T*)a, a_stride, row_token, (const T*)weight,
-            tile_expert, n_out, k_in, act);
+            tile_expert, n_out, k_in, act, row_scale);
         VLA_SEQ_HIP_CHECK(hipGetLastError());
         return VLA_OK;
       }
     }
     grouped_linear_kernel<S, SO><<<dim3(max_tiles, (n_out + kWave - 1) / kWave), 256, 0, st>>>(
         (typename SO::T*)out, out_stride, (const T*)a, a_stride, row_token, (const T*)weight,
-        tile_expert, n_out, k_in, act);
+        tile_expert, n_out, k_in, act, row_scale);
     VLA_SEQ_HIP_CHECK(hipGetLastError());
     return VLA_OK;
   });
@@ -594,7 +619,7 @@ extern "C" int vla_seq_moe_combine(float* out, const float* y, const int* pair_r
                                    const float* shared_y, const float* shared_gate, int num_tokens,
                                    int width, int top, int dtype, void* stream) {
   if (num_tokens == 0) return VLA_OK;
-  if (!out || !y || !pair_row || !weights || !h || num_tokens < 0 || width <= 0 || top <= 0 ||
+  if (!out || !y || !pair_row || !h || num_tokens < 0 || width <= 0 || top <= 0 ||
       h_stride < width)
     return VLA_ERR_ARG;
   return with_dtype(dtype, [&](auto s) {

@@ -14,6 +14,7 @@ _MODELS: Dict[str, Tuple[str, str, str]] = {
     "Dopipel": ("vllm_legacy_amd.model.dopipel", "DopipelForCausalLM", "DopipelConfig"),
     "Lamosun": ("vllm_legacy_amd.model.lamosun", "LamosunForCausalLM", "LamosunConfig"),
     "Tekezen": ("vllm_legacy_amd.model.tekezen", "TekezenForCausalLM", "TekezenConfig"),
+    "Batatar": ("vllm_legacy_amd.model.batatar", "BatatarForCausalLM", "BatatarConfig"),
     # the synthetic-weight Llama stack behind the engine's model protocol
     "LlamaDecodeStack": ("vllm_legacy_amd.engine.llama_adapter", "PagedLlamaForEngine", "LlamaEngineConfig"),
 }

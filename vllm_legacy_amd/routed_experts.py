@@ -2,7 +2,9 @@
 
 Router: z = W_r h (+ a bias) in fp32 over all routed experts, s = softmax(z); the `top` experts
 with the largest s + correction are chosen and weighted by their s renormalized to sum 1 (without a
-correction: the softmax over the chosen logits).  The last `identity` routed experts have no
+correction: the softmax over the chosen logits).  `score="sigmoid"` takes s = sigmoid(z) of each logit,
+`renormalize=False` the chosen s as they are, and `weight_input=True` lets a choice's weight multiply
+its expert's input instead of its output (the fp32 sums of W_gate h and W_up h are scaled).  The last `identity` routed experts have no
 weights: their output is the token's input.  An expert is W_down act(W_up h), or, `gated`,
 W_down (act(W_gate h) * W_up h); with act "clamped_glu" the gated form is
 g sigmoid(alpha g) (u + shift), g = min(W_gate h, limit), u = clamp(W_up h, -limit, limit).  An
@@ -40,8 +42,14 @@ class RoutedExperts(nn.Module):
                  shared_ff: int = 0, act: str = "relu2", shared_act: Optional[str] = None,
                  dtype=torch.bfloat16, device=None, gated: bool = False, router_bias: bool = False,
                  act_limit: float = 0.0, act_alpha: float = 1.702, act_shift: float = 1.0,
-                 shared_gated: bool = False, shared_limit: float = 0.0) -> None:
+                 shared_gated: bool = False, shared_limit: float = 0.0, score: str = "softmax",
+                 renormalize: bool = True, weight_input: bool = False) -> None:
         super().__init__()
+        if score not in ops.MOE_SCORE:
+            raise ValueError(f"unknown router score {score!r}")
+        if weight_input and num_identity:
+            raise ValueError("identity experts have no product to weight the input of")
+        self.score, self.renormalize, self.weight_input = score, bool(renormalize), bool(weight_input)
         if act == "clamped_glu" and not (gated and act_limit > 0):
             raise ValueError("clamped_glu needs gated experts and a limit")
         if shared_gated and shared_ff and (shared_act or act) == "clamped_glu" and not shared_limit > 0:
@@ -128,17 +136,23 @@ class RoutedExperts(nn.Module):
             logits = torch.mm(h if h.dtype == torch.float32 else h.float(), self.router_rows().t())
         experts, weights, sg = ops.moe_route(h, self.router.data, self.correction.data,
                                              None if self.shared_gate is None else self.shared_gate.data, self.top, logits,
-                                             None if self.router_bias is None else self.router_bias.data)
+                                             None if self.router_bias is None else self.router_bias.data,
+                                             self.score, self.renormalize)
         if self.num_experts:
-            pair_row, row_token, tile_expert = ops.moe_plan(experts, self.num_experts)
+            row_scale = None
+            if self.weight_input:
+                pair_row, row_token, tile_expert, row_scale = ops.moe_plan(experts, self.num_experts, weights)
+                weights = None
+            else:
+                pair_row, row_token, tile_expert = ops.moe_plan(experts, self.num_experts)
             rows = row_token.numel()
             u = torch.empty((rows, self.expert_ff), dtype=h.dtype, device=h.device)
             if self.gated:
                 both = torch.empty((rows, 2 * self.expert_ff), dtype=h.dtype, device=h.device)
-                ops.grouped_linear(both, h, row_token, self.w_up.data, tile_expert)
+                ops.grouped_linear(both, h, row_token, self.w_up.data, tile_expert, row_scale=row_scale)
                 self._glu(u, both, self.expert_ff, self.act, self.act_limit)
             else:
-                ops.grouped_linear(u, h, row_token, self.w_up.data, tile_expert, self.act)
+                ops.grouped_linear(u, h, row_token, self.w_up.data, tile_expert, self.act, row_scale)
             y = torch.empty((rows, self.width), dtype=torch.float32, device=h.device)
             ops.grouped_linear(y, u, None, self.w_down.data, tile_expert)
         else:   # identity experts only
