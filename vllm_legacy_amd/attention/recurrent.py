@@ -247,7 +247,7 @@ class ConstantDecayRecurrence(nn.Module):
             raise ValueError("one decay in [0, 1] per head is needed")
         self.heads, self.dim, self.vdim, self.eps, self.act = heads, dim, vdim, float(eps), act
         # a decay of 0 forgets everything: a finite stand-in for its logarithm keeps sums of it finite
-        logs = [max(math.log(d), -1e30) if d > 0.0 else -1e30 for d in map(float, decay)]
+        logs = [max(math.log(d), -1e4) if d > 0.0 else -1e4 for d in map(float, decay)]
         self.register_buffer("log_decay", torch.tensor(logs, dtype=torch.float64).to(torch.float32).to(device),
                              persistent=False)
         self.norm_weight = nn.Parameter(torch.ones(heads * vdim, dtype=torch.float32, device=device), requires_grad=False)

@@ -8,7 +8,8 @@
 //   o_i = e^(c_i) S^T q_i + sum_(j <= i) e^(c_i - c_j) w_j (q_i . k_j) v_j + skip v_i
 //   S  <- e^(c_last) S + sum_j e^(c_last - c_j) w_j k_j v_j^T
 // are three matrix products per block around the products P = Q K^T; every exponent is a sum of
-// g <= 0, so nothing overflows.  All of it runs on fp32 matrix cores (16x16x4): nothing is rounded
+// g <= 0, so nothing overflows; c is summed in fp64 and kept as two fp32 numbers, so that differences of
+// large sums stay exact to fp32.  All of it runs on fp32 matrix cores (16x16x4): nothing is rounded
 // below fp32 after it has been read.  Layout, lane = (g, c) = (lane >> 4, lane & 15):
 //   A operand  lane: row c, contraction index g       B operand  lane: column c, contraction index g
 //   result     lane: column c, rows 4 g .. 4 g + 3
@@ -201,7 +202,7 @@ __device__ __forceinline__ bool find_piece(const DecayScan& a, int z, int& b, in
 template <int DB, int NV, bool STATE_ONLY>
 constexpr size_t block_lds_floats() {
   return (size_t)kBlock * ((STATE_ONLY ? 1 : 2) * (16 * DB + 4) + (64 * NV + 4) + (STATE_ONLY ? 0 : kBlock + 4)) +
-         4 * kBlock;
+         5 * kBlock;
 }
 
 template <int DB, int NV, bool W16, bool STATE_ONLY>
@@ -211,8 +212,8 @@ __global__ __launch_bounds__(256) void decay_block_kernel(DecayScan a) {
   extern __shared__ __align__(16) float lds[];
   float* k_lds = lds;                                   // [64][KR]
   float* v_lds = k_lds + kBlock * KR;                   // [64][VR]
-  float* num = v_lds + kBlock * VR;                     // c | w | e^c | e^(c_last - c) w
-  float* q_lds = num + 4 * kBlock;                      // [64][KR]
+  float* num = v_lds + kBlock * VR;                     // c | w | e^c | e^(c_last - c) w | c's low part
+  float* q_lds = num + 5 * kBlock;                      // [64][KR]
   float* p_lds = q_lds + kBlock * KR;                   // [64][PR]
   const int h = blockIdx.x, v0 = blockIdx.y * VB, z = blockIdx.z;
   int b, piece;
@@ -245,7 +246,7 @@ __global__ __launch_bounds__(256) void decay_block_kernel(DecayScan a) {
         s[nv][db][r] = from != nullptr && d < D && v < V ? from[(int64_t)d * V + v] : 0.f;
       }
   const float skip = a.skip != nullptr && !STATE_ONLY ? a.skip[h] : 0.f;
-  float log_total = 0.f;
+  double log_total = 0.0;
 
   Piece<W16> pq[NQ], pk[NQ], pv[NVP];
   float row_g = 0.f, row_w = 0.f;
@@ -271,17 +272,18 @@ __global__ __launch_bounds__(256) void decay_block_kernel(DecayScan a) {
   };
   auto land = [&]() {
     if (w == 0) {
-      float cs = row_g;                                 // inclusive sum over the 64 rows
+      double cs = row_g;                                // inclusive sum over the 64 rows
 #pragma unroll
       for (int m = 1; m < 64; m <<= 1) {
-        const float other = __shfl_up(cs, m, 64);
-        cs += lane >= m ? other : 0.f;
+        const double other = __shfl_up(cs, m, 64);
+        cs += lane >= m ? other : 0.0;
       }
-      const float end = __shfl(cs, 63, 64);
-      num[lane] = cs;
+      const double end = __shfl(cs, 63, 64);
+      num[lane] = (float)cs;
       num[kBlock + lane] = row_w;
-      num[2 * kBlock + lane] = expf(cs);
-      num[3 * kBlock + lane] = expf(end - cs) * row_w;
+      num[2 * kBlock + lane] = expf((float)cs);
+      num[3 * kBlock + lane] = expf(fminf((float)(end - cs), 0.f)) * row_w;
+      num[4 * kBlock + lane] = (float)(cs - (double)(float)cs);
     }
 #pragma unroll
     for (int u = 0; u < NQ; ++u) {
@@ -317,11 +319,12 @@ __global__ __launch_bounds__(256) void decay_block_kernel(DecayScan a) {
           for (int i = 0; i < 4; ++i) acc = mfma4(qa[i], ka[i], acc);
         }
         const int j = 16 * jb + c;
-        const float cj = num[j], wj = num[kBlock + j];
+        const float cj = num[j], lj = num[4 * kBlock + j], wj = num[kBlock + j];
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
           const int i = 16 * ib + 4 * g + r;
-          p_lds[i * PR + j] = j <= i ? acc[r] * (expf(num[i] - cj) * wj) : 0.f;
+          const float diff = fminf((num[i] - cj) + (num[4 * kBlock + i] - lj), 0.f);
+          p_lds[i * PR + j] = j <= i ? acc[r] * (expf(diff) * wj) : 0.f;
         }
       }
       __syncthreads();
@@ -375,7 +378,7 @@ __global__ __launch_bounds__(256) void decay_block_kernel(DecayScan a) {
       }
     }
     const float e_last = num[2 * kBlock + kBlock - 1];
-    log_total += num[kBlock - 1];
+    log_total += (double)num[kBlock - 1] + (double)num[5 * kBlock - 1];
 #pragma unroll
     for (int kb = 0; kb < 4; ++kb) {
       const f32x4 tw = *reinterpret_cast<const f32x4*>(num + 3 * kBlock + 16 * kb + 4 * g);
@@ -407,7 +410,7 @@ __global__ __launch_bounds__(256) void decay_block_kernel(DecayScan a) {
   float* to;
   if (STATE_ONLY) {
     to = a.piece_state + ((int64_t)z * a.heads + h) * state_size;
-    if (tid == 0 && blockIdx.y == 0) a.piece_decay[(int64_t)z * a.heads + h] = expf(log_total);
+    if (tid == 0 && blockIdx.y == 0) a.piece_decay[(int64_t)z * a.heads + h] = expf((float)log_total);
   } else {
     if (!last) return;
     to = a.state + ((int64_t)a.state_slots[b] * a.heads + h) * state_size;
