@@ -543,6 +543,47 @@ def test_a_far_token_is_carried_by_a_slow_decay(cuts):
     assert float(got[-1, 1].abs().max()) < 1e-6
 
 
+@pytest.mark.parametrize("dtypes", [(torch.float32, torch.float32), (torch.bfloat16, torch.bfloat16), (torch.float32, torch.bfloat16),
+                                    (torch.bfloat16, torch.float32)])
+@pytest.mark.parametrize("channels,taps", [(48, 4), (64, 3), (24, 2), (40, 1), (50, 4), (32, 7), (2056, 4)])
+def test_short_convolution_across_cuts_and_batches(dtypes, channels, taps):
+    """Aligned rows (runs of rows per thread) and any others; sequences of unequal lengths, single rows beside
+    portions, more than a thousand rows at once, a slot taken over; both kernels agree with the reference."""
+    from vllm_legacy_amd import _seq_ops as ops
+    from vllm_legacy_amd.layers import ShortConv
+    din, dout = dtypes
+    conv = ShortConv(channels, taps, True, "silu", DEV)
+    w, b = rnd((channels, taps), 1), rnd((channels, ), 2)
+    conv.weight.data, conv.bias.data = w.to(DEV), b.to(DEV)
+    lens = {"a": 1200 if channels == 48 else 60, "b": 7, "c": 33, "d": 12}
+    seqs = {k: rnd((n, channels), 3 + i).to(din) for i, (k, n) in enumerate(lens.items())}
+    want = {k: R.short_conv(u.to(F), w.to(F), b.to(F)) for k, u in seqs.items()}
+    slots = {"a": 0, "b": 1, "c": 2, "d": 1}
+    plan = [[("a", lens["a"] - 20), ("b", 2)], [("b", 1), ("a", 1), ("c", 1)], [("c", 1), ("b", 4), ("a", 9)],
+            [("a", 1), ("c", 1), ("d", 1)], [("d", 1)], [("d", 8), ("c", 30), ("a", 9)], [("d", 2)]]
+    for mode in (0, 1):
+        ops.set_short_conv_kernel(mode)
+        try:
+            state = torch.full((3, max(taps - 1, 0), channels), 5.0, device=DEV)
+            at, got = {k: 0 for k in seqs}, {k: [] for k in seqs}
+            for step in plan:
+                batch = make_batch([n for _, n in step], [at[k] for k, _ in step], 4, slots=[slots[k] for k, _ in step])
+                wide = torch.zeros((sum(n for _, n in step), channels + 8), dtype=din)
+                wide[:, 8:] = torch.cat([seqs[k][at[k]:at[k] + n] for k, n in step])
+                out = torch.empty((wide.shape[0], channels), dtype=dout, device=DEV)
+                conv(out, wide.to(DEV)[:, 8:], state if taps > 1 else None, batch)
+                lo = 0
+                for k, n in step:
+                    got[k].append(out[lo:lo + n].float().cpu())
+                    at[k] += n
+                    lo += n
+            assert at == lens
+            for k in seqs:
+                close(torch.cat(got[k]), want[k], 1e-6 if dout == torch.float32 else 6e-3, (mode, k))
+        finally:
+            ops.set_short_conv_kernel(0)
+
+
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
 @pytest.mark.parametrize("shape", [(4, 16, 8, 2, 2, 4), (6, 10, 14, 3, 5, 3), (3, 7, 5, 1, 7, 1), (2, 64, 32, 1, 1, 4)])
 def test_state_space_layer_across_cuts(dtype, shape):

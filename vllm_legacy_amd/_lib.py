@@ -66,7 +66,7 @@ SEQ_EXPORTS = [
     "vla_seq_latent_attention_tiles_supported", "vla_seq_latent_attention_scratch_floats", "vla_seq_set_latent_attention_kernel",
     "vla_seq_clamped_glu", "vla_seq_pair_hash_embed",
     "vla_seq_decay_scan", "vla_seq_decay_scan_scratch_floats", "vla_seq_set_decay_scan_kernel",
-    "vla_seq_gated_group_rms_norm",
+    "vla_seq_gated_group_rms_norm", "vla_seq_set_short_conv_kernel",
 ]
 _seq_lib = None
 
@@ -129,7 +129,8 @@ def seq_lib():
         L.vla_seq_moe_route.argtypes = [p, i64, p, p, i64, p, p, p, p, p, p, i, i, i, i, i, i, i, p]
         L.vla_seq_post_norm.argtypes = [p, f, p, i64, i, p, f, p, i, i, i, p]
         L.vla_seq_rms_norm_rows.argtypes = [p, i64, i, p, i64, i, p, f, i, i, p]
-        L.vla_seq_short_conv.argtypes = [p, i64, i, p, i64, i, p, p, p, p, p, p, p, i, i, i, i, i, i, p]
+        L.vla_seq_short_conv.argtypes = [p, i64, i, p, i64, i, p, p, p, p, p, p, p, i, i, i, i, i, i, i, p]
+        L.vla_seq_set_short_conv_kernel.argtypes = [i]
         L.vla_seq_gated_act_lookup.argtypes = [p, i64, i, p, i64, i, p, i64, i, p, i, i, i, i, i, p]
         L.vla_seq_embed_scaled.argtypes = [p, p, p, f, i, i, i, i, p]
         L.vla_seq_softcap.argtypes = [p, i64, f, p]

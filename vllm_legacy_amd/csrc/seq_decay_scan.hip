@@ -17,7 +17,9 @@
 // step i of block kb, and what a lane holds of a result with rows 16 db + 4 g + i is the B operand of
 // that step: a wave keeps S of its value columns in registers as a result and uses it as an operand
 // where it lies.  A workgroup walks one run (or piece of a run) of one head for 64 or 128 value
-// columns, 16 or 32 per wave; rows come one block ahead through registers into LDS.
+// columns, 16 per wave; rows come one block ahead through registers into LDS.  bfloat16 queries and
+// keys without an activation stay bfloat16 there (half the LDS: two workgroups per CU) and P comes from
+// the bfloat16 products, which are exact in fp32 as well; everything else sees them as fp32.
 //
 // Long runs are cut into pieces of VLA_DECAY_SCAN_PIECE rows: (1) every piece but the last forms the
 // state its own rows leave from a zero state; (2) a chain over a sequence's pieces turns these
@@ -29,6 +31,7 @@
 // gated_group_rms_norm: what follows such a recurrence, per token: gate and RMS norm over equal
 // parts of the concatenated heads.
 #include <atomic>
+#include <type_traits>
 
 #include "seq_common.h"
 
@@ -199,22 +202,35 @@ __device__ __forceinline__ bool find_piece(const DecayScan& a, int z, int& b, in
   return piece >= 0 && (int64_t)piece * a.piece_rows < a.query_start_loc[b + 1] - a.query_start_loc[b];
 }
 
-template <int DB, int NV, bool STATE_ONLY>
+// How a block kernel reads and keeps its rows
+enum RowKind {
+  kRowsF32,      // fp32 in memory and in LDS
+  kRows16,       // 16-bit in memory, fp32 in LDS (after the activation)
+  kRowsBf16      // queries and keys bfloat16 in LDS too (no activation)
+};
+
+template <int DB, int WAVES, RowKind KIND, bool STATE_ONLY>
 constexpr size_t block_lds_floats() {
-  return (size_t)kBlock * ((STATE_ONLY ? 1 : 2) * (16 * DB + 4) + (64 * NV + 4) + (STATE_ONLY ? 0 : kBlock + 4)) +
-         5 * kBlock;
+  constexpr int DP = 16 * DB, QK = KIND == kRowsBf16 ? (DP + 8) / 2 : DP + 4;     // floats per query / key row
+  return (size_t)kBlock * ((STATE_ONLY ? 1 : 2) * QK + (16 * WAVES + 4) + (STATE_ONLY ? 0 : kBlock + 4)) + 5 * kBlock;
 }
 
-template <int DB, int NV, bool W16, bool STATE_ONLY>
-__global__ __launch_bounds__(256) void decay_block_kernel(DecayScan a) {
-  constexpr int DP = 16 * DB, KR = DP + 4, VB = 64 * NV, VR = VB + 4, PR = kBlock + 4;
-  constexpr int NQ = (DP * kBlock / 8 + 255) / 256, NVP = VB * kBlock / 8 / 256;   // pieces per thread
+template <int DB, int WAVES, RowKind KIND, bool STATE_ONLY>
+__global__ __launch_bounds__(64 * WAVES) void decay_block_kernel(DecayScan a) {
+  constexpr bool W16 = KIND != kRowsF32, QK16 = KIND == kRowsBf16;
+  constexpr int THREADS = 64 * WAVES;
+  constexpr int DP = 16 * DB, KR = QK16 ? DP + 8 : DP + 4;      // elements of a query / key row
+  constexpr int QK_FLOATS = QK16 ? KR / 2 : KR;
+  constexpr int VB = 16 * WAVES, VR = VB + 4, PR = kBlock + 4;
+  constexpr int NQ = (DP * kBlock / 8 + THREADS - 1) / THREADS;         // pieces of eight values per thread
+  constexpr int NVP = VB * kBlock / 8 / THREADS;
+  using E = typename std::conditional<QK16, uint16_t, float>::type;
   extern __shared__ __align__(16) float lds[];
-  float* k_lds = lds;                                   // [64][KR]
-  float* v_lds = k_lds + kBlock * KR;                   // [64][VR]
+  E* k_lds = reinterpret_cast<E*>(lds);                 // [64][KR]
+  float* v_lds = lds + kBlock * QK_FLOATS;              // [64][VR]
   float* num = v_lds + kBlock * VR;                     // c | w | e^c | e^(c_last - c) w | c's low part
-  float* q_lds = num + 5 * kBlock;                      // [64][KR]
-  float* p_lds = q_lds + kBlock * KR;                   // [64][PR]
+  E* q_lds = reinterpret_cast<E*>(num + 5 * kBlock);    // [64][KR]
+  float* p_lds = num + 5 * kBlock + kBlock * QK_FLOATS; // [64][PR]
   const int h = blockIdx.x, v0 = blockIdx.y * VB, z = blockIdx.z;
   int b, piece;
   if (!find_piece(a, z, b, piece)) return;
@@ -227,6 +243,7 @@ __global__ __launch_bounds__(256) void decay_block_kernel(DecayScan a) {
   const int t_begin = a.query_start_loc[b] + first, t_end = last ? a.query_start_loc[b + 1] : t_begin + a.piece_rows;
   const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6, g = lane >> 4, c = lane & 15;
   const int D = a.dim, V = a.vdim, hg = h / (a.heads / a.groups);
+  const int v_mine = v0 + 16 * w + c;                   // this lane's value column
   const int64_t state_size = (int64_t)D * V;
   const float* from = nullptr;
   if (!STATE_ONLY) {
@@ -235,16 +252,14 @@ __global__ __launch_bounds__(256) void decay_block_kernel(DecayScan a) {
     else if (a.context_lens[b] > 0)
       from = a.state + ((int64_t)a.state_slots[b] * a.heads + h) * state_size;
   }
-  f32x4 s[NV][DB];
+  f32x4 s[DB];
 #pragma unroll
-  for (int nv = 0; nv < NV; ++nv)
+  for (int db = 0; db < DB; ++db)
 #pragma unroll
-    for (int db = 0; db < DB; ++db)
-#pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int d = 16 * db + 4 * g + r, v = v0 + 16 * (w * NV + nv) + c;
-        s[nv][db][r] = from != nullptr && d < D && v < V ? from[(int64_t)d * V + v] : 0.f;
-      }
+    for (int r = 0; r < 4; ++r) {
+      const int d = 16 * db + 4 * g + r;
+      s[db][r] = from != nullptr && d < D && v_mine < V ? from[(int64_t)d * V + v_mine] : 0.f;
+    }
   const float skip = a.skip != nullptr && !STATE_ONLY ? a.skip[h] : 0.f;
   double log_total = 0.0;
 
@@ -254,7 +269,7 @@ __global__ __launch_bounds__(256) void decay_block_kernel(DecayScan a) {
     const int n = min(kBlock, t_end - t0);
 #pragma unroll
     for (int u = 0; u < NQ; ++u) {
-      const int i = tid + 256 * u, r = i / (DP / 8), d = 8 * (i % (DP / 8));
+      const int i = tid + THREADS * u, r = i / (DP / 8), d = 8 * (i % (DP / 8));
       const bool row = r < n;
       pk[u] = read_piece<W16>(a.k, (int64_t)(t0 + r) * a.k_stride + (int64_t)hg * D, d, D, row, a.vec_k);
       if (!STATE_ONLY)
@@ -262,13 +277,19 @@ __global__ __launch_bounds__(256) void decay_block_kernel(DecayScan a) {
     }
 #pragma unroll
     for (int u = 0; u < NVP; ++u) {
-      const int i = tid + 256 * u, r = i / (VB / 8), d = v0 + 8 * (i % (VB / 8));
+      const int i = tid + THREADS * u, r = i / (VB / 8), d = v0 + 8 * (i % (VB / 8));
       pv[u] = read_piece<W16>(a.v, (int64_t)(t0 + r) * a.v_stride + (int64_t)h * V, d, V, r < n, a.vec_v);
     }
     if (tid < kBlock) {
       row_g = row_w = 0.f;
       if (tid < n) row_decay(a, t0 + tid, h, row_g, row_w);
     }
+  };
+  auto land_qk = [&](E* dst, const Piece<W16>& p) {
+    if constexpr (QK16)
+      *reinterpret_cast<u32x4*>(dst) = p.x;
+    else
+      land_piece<W16>(dst, p, a.act, a.dtype);
   };
   auto land = [&]() {
     if (w == 0) {
@@ -287,16 +308,32 @@ __global__ __launch_bounds__(256) void decay_block_kernel(DecayScan a) {
     }
 #pragma unroll
     for (int u = 0; u < NQ; ++u) {
-      const int i = tid + 256 * u, r = i / (DP / 8), d = 8 * (i % (DP / 8));
-      if (NQ * 256 * 8 != DP * kBlock && r >= kBlock) continue;
-      land_piece<W16>(k_lds + r * KR + d, pk[u], a.act, a.dtype);
-      if (!STATE_ONLY) land_piece<W16>(q_lds + r * KR + d, pq[u], a.act, a.dtype);
+      const int i = tid + THREADS * u, r = i / (DP / 8), d = 8 * (i % (DP / 8));
+      if (DP * kBlock / 8 % THREADS != 0 && r >= kBlock) continue;
+      land_qk(k_lds + r * KR + d, pk[u]);
+      if (!STATE_ONLY) land_qk(q_lds + r * KR + d, pq[u]);
     }
 #pragma unroll
     for (int u = 0; u < NVP; ++u) {
-      const int i = tid + 256 * u, r = i / (VB / 8), d = 8 * (i % (VB / 8));
+      const int i = tid + THREADS * u, r = i / (VB / 8), d = 8 * (i % (VB / 8));
       land_piece<W16>(v_lds + r * VR + d, pv[u], a.act, a.dtype);
     }
+  };
+  // four consecutive values of a query / key row, and one, as fp32
+  auto four = [&](const E* src) {
+    if constexpr (QK16) {
+      const u32x2 x = *reinterpret_cast<const u32x2*>(src);
+      return f32x4{__builtin_bit_cast(float, x[0] << 16), __builtin_bit_cast(float, x[0] & 0xffff0000u),
+                   __builtin_bit_cast(float, x[1] << 16), __builtin_bit_cast(float, x[1] & 0xffff0000u)};
+    } else {
+      return *reinterpret_cast<const f32x4*>(src);
+    }
+  };
+  auto one = [&](const E* src) {
+    if constexpr (QK16)
+      return __builtin_bit_cast(float, (uint32_t)*src << 16);
+    else
+      return *src;
   };
 
   fetch(t_begin);
@@ -307,16 +344,26 @@ __global__ __launch_bounds__(256) void decay_block_kernel(DecayScan a) {
     if (t0 + kBlock < t_end) fetch(t0 + kBlock);
     if constexpr (!STATE_ONLY) {
       // P_ij = (q_i . k_j) e^(c_i - c_j) w_j for j <= i: ten 16 x 16 tiles, dealt to the waves
-      for (int ti = w; ti < 10; ti += 4) {
+      for (int ti = w; ti < 10; ti += WAVES) {
         const int ib = ti < 1 ? 0 : ti < 3 ? 1 : ti < 6 ? 2 : 3, jb = ti - ib * (ib + 1) / 2;
         if (16 * ib >= n) break;
         f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+        if constexpr (QK16) {
 #pragma unroll
-        for (int kb = 0; kb < DB; ++kb) {
-          const f32x4 qa = *reinterpret_cast<const f32x4*>(q_lds + (16 * ib + c) * KR + 16 * kb + 4 * g);
-          const f32x4 ka = *reinterpret_cast<const f32x4*>(k_lds + (16 * jb + c) * KR + 16 * kb + 4 * g);
+          for (int kb = 0; kb < DP / 32; ++kb) {
+            const u32x4 qa = *reinterpret_cast<const u32x4*>(q_lds + (16 * ib + c) * KR + 32 * kb + 8 * g);
+            const u32x4 ka = *reinterpret_cast<const u32x4*>(k_lds + (16 * jb + c) * KR + 32 * kb + 8 * g);
+            acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, qa), __builtin_bit_cast(bf16x8, ka),
+                                                          acc, 0, 0, 0);
+          }
+        } else {
 #pragma unroll
-          for (int i = 0; i < 4; ++i) acc = mfma4(qa[i], ka[i], acc);
+          for (int kb = 0; kb < DB; ++kb) {
+            const f32x4 qa = four(q_lds + (16 * ib + c) * KR + 16 * kb + 4 * g);
+            const f32x4 ka = four(k_lds + (16 * jb + c) * KR + 16 * kb + 4 * g);
+#pragma unroll
+            for (int i = 0; i < 4; ++i) acc = mfma4(qa[i], ka[i], acc);
+          }
         }
         const int j = 16 * jb + c;
         const float cj = num[j], lj = num[4 * kBlock + j], wj = num[kBlock + j];
@@ -330,49 +377,35 @@ __global__ __launch_bounds__(256) void decay_block_kernel(DecayScan a) {
       __syncthreads();
     }
     // this wave's value columns as B operands: rows 16 kb + 4 g + i
-    float vf[NV][4][4];
+    float vf[4][4];
 #pragma unroll
-    for (int nv = 0; nv < NV; ++nv)
+    for (int kb = 0; kb < 4; ++kb)
 #pragma unroll
-      for (int kb = 0; kb < 4; ++kb)
-#pragma unroll
-        for (int i = 0; i < 4; ++i) vf[nv][kb][i] = v_lds[(16 * kb + 4 * g + i) * VR + 16 * (w * NV + nv) + c];
+      for (int i = 0; i < 4; ++i) vf[kb][i] = v_lds[(16 * kb + 4 * g + i) * VR + 16 * w + c];
     if constexpr (!STATE_ONLY) {
 #pragma unroll
       for (int rb = 0; rb < 4; ++rb) {
         if (16 * rb < n) {
-          f32x4 acc[NV];
-#pragma unroll
-          for (int nv = 0; nv < NV; ++nv) acc[nv] = f32x4{0.f, 0.f, 0.f, 0.f};
+          f32x4 acc = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
           for (int db = 0; db < DB; ++db) {
-            const f32x4 qa = *reinterpret_cast<const f32x4*>(q_lds + (16 * rb + c) * KR + 16 * db + 4 * g);
+            const f32x4 qa = four(q_lds + (16 * rb + c) * KR + 16 * db + 4 * g);
 #pragma unroll
-            for (int i = 0; i < 4; ++i)
-#pragma unroll
-              for (int nv = 0; nv < NV; ++nv) acc[nv] = mfma4(qa[i], s[nv][db][i], acc[nv]);
+            for (int i = 0; i < 4; ++i) acc = mfma4(qa[i], s[db][i], acc);
           }
           const f32x4 ec = *reinterpret_cast<const f32x4*>(num + 2 * kBlock + 16 * rb + 4 * g);
 #pragma unroll
-          for (int nv = 0; nv < NV; ++nv)
-#pragma unroll
-            for (int r = 0; r < 4; ++r) acc[nv][r] = acc[nv][r] * ec[r] + skip * vf[nv][rb][r];
+          for (int r = 0; r < 4; ++r) acc[r] = acc[r] * ec[r] + skip * vf[rb][r];
 #pragma unroll
           for (int kb = 0; kb <= rb; ++kb) {
             const f32x4 pa = *reinterpret_cast<const f32x4*>(p_lds + (16 * rb + c) * PR + 16 * kb + 4 * g);
 #pragma unroll
-            for (int i = 0; i < 4; ++i)
-#pragma unroll
-              for (int nv = 0; nv < NV; ++nv) acc[nv] = mfma4(pa[i], vf[nv][kb][i], acc[nv]);
+            for (int i = 0; i < 4; ++i) acc = mfma4(pa[i], vf[kb][i], acc);
           }
 #pragma unroll
-          for (int nv = 0; nv < NV; ++nv) {
-            const int v = v0 + 16 * (w * NV + nv) + c;
-#pragma unroll
-            for (int r = 0; r < 4; ++r) {
-              const int i = 16 * rb + 4 * g + r;
-              if (i < n && v < V) a.o[((int64_t)(t0 + i) * a.heads + h) * V + v] = acc[nv][r];
-            }
+          for (int r = 0; r < 4; ++r) {
+            const int i = 16 * rb + 4 * g + r;
+            if (i < n && v_mine < V) a.o[((int64_t)(t0 + i) * a.heads + h) * V + v_mine] = acc[r];
           }
         }
       }
@@ -383,25 +416,18 @@ __global__ __launch_bounds__(256) void decay_block_kernel(DecayScan a) {
     for (int kb = 0; kb < 4; ++kb) {
       const f32x4 tw = *reinterpret_cast<const f32x4*>(num + 3 * kBlock + 16 * kb + 4 * g);
 #pragma unroll
-      for (int nv = 0; nv < NV; ++nv)
-#pragma unroll
-        for (int i = 0; i < 4; ++i) vf[nv][kb][i] *= tw[i];
+      for (int i = 0; i < 4; ++i) vf[kb][i] *= tw[i];
     }
 #pragma unroll
     for (int db = 0; db < DB; ++db) {
 #pragma unroll
-      for (int nv = 0; nv < NV; ++nv)
-#pragma unroll
-        for (int r = 0; r < 4; ++r) s[nv][db][r] *= e_last;
+      for (int r = 0; r < 4; ++r) s[db][r] *= e_last;
 #pragma unroll
       for (int kb = 0; kb < 4; ++kb) {
         if (16 * kb < n) {
 #pragma unroll
-          for (int i = 0; i < 4; ++i) {
-            const float ka = k_lds[(16 * kb + 4 * g + i) * KR + 16 * db + c];
-#pragma unroll
-            for (int nv = 0; nv < NV; ++nv) s[nv][db] = mfma4(ka, vf[nv][kb][i], s[nv][db]);
-          }
+          for (int i = 0; i < 4; ++i)
+            s[db] = mfma4(one(k_lds + (16 * kb + 4 * g + i) * KR + 16 * db + c), vf[kb][i], s[db]);
         }
       }
     }
@@ -416,14 +442,12 @@ __global__ __launch_bounds__(256) void decay_block_kernel(DecayScan a) {
     to = a.state + ((int64_t)a.state_slots[b] * a.heads + h) * state_size;
   }
 #pragma unroll
-  for (int nv = 0; nv < NV; ++nv)
+  for (int db = 0; db < DB; ++db)
 #pragma unroll
-    for (int db = 0; db < DB; ++db)
-#pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int d = 16 * db + 4 * g + r, v = v0 + 16 * (w * NV + nv) + c;
-        if (d < D && v < V) to[(int64_t)d * V + v] = s[nv][db][r];
-      }
+    for (int r = 0; r < 4; ++r) {
+      const int d = 16 * db + 4 * g + r;
+      if (d < D && v_mine < V) to[(int64_t)d * V + v_mine] = s[db][r];
+    }
 }
 
 // Over one sequence's pieces: what piece i leaves from zero (in its slot) becomes what it starts from.
@@ -630,42 +654,42 @@ __global__ __launch_bounds__(256) void gated_group_rms_norm_kernel(
   }
 }
 
-template <int DB, int NV, bool W16, bool STATE_ONLY>
+template <int DB, int WAVES, RowKind KIND, bool STATE_ONLY>
 int launch_block(const DecayScan& a, int pieces, hipStream_t stream) {
-  constexpr size_t lds = block_lds_floats<DB, NV, STATE_ONLY>() * sizeof(float);
+  constexpr size_t lds = block_lds_floats<DB, WAVES, KIND, STATE_ONLY>() * sizeof(float);
   static std::atomic<bool> allowed{false};              // raised once per kernel, not per launch
   if (lds > 64 * 1024 && !allowed.load(std::memory_order_relaxed)) {
     VLA_SEQ_HIP_CHECK(hipFuncSetAttribute(
-        reinterpret_cast<const void*>(&decay_block_kernel<DB, NV, W16, STATE_ONLY>),
+        reinterpret_cast<const void*>(&decay_block_kernel<DB, WAVES, KIND, STATE_ONLY>),
         hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds));
     allowed.store(true, std::memory_order_relaxed);
   }
-  const dim3 grid(a.heads, (a.vdim + 64 * NV - 1) / (64 * NV), pieces);
-  decay_block_kernel<DB, NV, W16, STATE_ONLY><<<grid, 256, lds, stream>>>(a);
+  const dim3 grid(a.heads, (a.vdim + 16 * WAVES - 1) / (16 * WAVES), pieces);
+  decay_block_kernel<DB, WAVES, KIND, STATE_ONLY><<<grid, 64 * WAVES, lds, stream>>>(a);
   VLA_SEQ_HIP_CHECK(hipGetLastError());
   return VLA_OK;
 }
 
-template <int DB, int NV, bool W16>
-int launch_blocks(DecayScan a, int pieces, hipStream_t stream) {
+template <int DB, int WAVES, RowKind KIND>
+int launch_blocks(const DecayScan& a, int pieces, hipStream_t stream) {
   if (a.piece_rows > 0) {
-    const int rc = launch_block<DB, NV, W16, true>(a, pieces, stream);
+    const int rc = launch_block<DB, WAVES, KIND, true>(a, pieces, stream);
     if (rc != VLA_OK) return rc;
     const int64_t size = (int64_t)a.dim * a.vdim;
     decay_chain_kernel<<<dim3((unsigned)((size + 255) / 256), a.heads, a.num_seqs), 256, 0, stream>>>(a);
     VLA_SEQ_HIP_CHECK(hipGetLastError());
   }
-  return launch_block<DB, NV, W16, false>(a, pieces, stream);
+  return launch_block<DB, WAVES, KIND, false>(a, pieces, stream);
 }
 
-template <bool W16>
+template <RowKind KIND>
 int launch_by_size(const DecayScan& a, int pieces, hipStream_t stream) {
   const bool wide = a.vdim > 64;
   switch ((a.dim + 31) / 32) {
-    case 1: return wide ? launch_blocks<2, 2, W16>(a, pieces, stream) : launch_blocks<2, 1, W16>(a, pieces, stream);
-    case 2: return wide ? launch_blocks<4, 2, W16>(a, pieces, stream) : launch_blocks<4, 1, W16>(a, pieces, stream);
-    case 3: return wide ? launch_blocks<6, 2, W16>(a, pieces, stream) : launch_blocks<6, 1, W16>(a, pieces, stream);
-    case 4: return wide ? launch_blocks<8, 2, W16>(a, pieces, stream) : launch_blocks<8, 1, W16>(a, pieces, stream);
+    case 1: return wide ? launch_blocks<2, 8, KIND>(a, pieces, stream) : launch_blocks<2, 4, KIND>(a, pieces, stream);
+    case 2: return wide ? launch_blocks<4, 8, KIND>(a, pieces, stream) : launch_blocks<4, 4, KIND>(a, pieces, stream);
+    case 3: return wide ? launch_blocks<6, 8, KIND>(a, pieces, stream) : launch_blocks<6, 4, KIND>(a, pieces, stream);
+    case 4: return wide ? launch_blocks<8, 8, KIND>(a, pieces, stream) : launch_blocks<8, 4, KIND>(a, pieces, stream);
     default: return VLA_ERR_HEAD_SIZE;
   }
 }
@@ -779,7 +803,9 @@ extern "C" int vla_seq_decay_scan(float* o, const void* q, int64_t q_stride, con
     VLA_SEQ_HIP_CHECK(hipGetLastError());
   }
   if (!blocks) return VLA_OK;
-  return dtype == VLA_F32 ? launch_by_size<false>(a, pieces, st) : launch_by_size<true>(a, pieces, st);
+  if (dtype == VLA_F32) return launch_by_size<kRowsF32>(a, pieces, st);
+  if (dtype == VLA_BF16 && act == VLA_ACT_NONE) return launch_by_size<kRowsBf16>(a, pieces, st);
+  return launch_by_size<kRows16>(a, pieces, st);
 }
 
 extern "C" int vla_seq_gated_group_rms_norm(void* out, int64_t out_stride, const float* o,

@@ -8,12 +8,15 @@
 //   embed_scaled      table[id] * scale as the fp32 stream
 //   softcap           z <- cap * tanh(z / cap)
 // One workgroup per row, fp32 arithmetic throughout; rows are read / written in the types named.
+#include <atomic>
+
 #include "seq_common.h"
 
 namespace vla {
 namespace seq {
 namespace {
 
+std::atomic<int> g_conv_kernel{0};
 constexpr int kThreads = 256;
 constexpr int kKeep = 8;          // row elements a thread keeps in registers (rows up to 2048)
 constexpr int kMaxTaps = 32;
@@ -116,17 +119,129 @@ __global__ __launch_bounds__(kThreads) void short_conv_kernel(
   }
 }
 
+// Two to four taps, rows and channels in whole 16-byte pieces: a thread takes 16 bytes of channels
+// through `run` consecutive rows of the step and keeps the taps - 1 inputs before the current row in
+// registers, so a row is read once per run and taps - 1 times more at its start.  Where a sequence
+// brings a single row (decode steps) the thread that has it also leaves the sequence's new state: no
+// other thread reads that slot.
+template <class S, int VC>
+__device__ __forceinline__ void load_channels(const typename S::T* p, float (&x)[VC]) {
+  if constexpr (sizeof(typename S::T) == 2) {
+    const u32x4 got = *reinterpret_cast<const u32x4*>(p);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      x[2 * e] = lo16<S>(got[e]);
+      x[2 * e + 1] = hi16<S>(got[e]);
+    }
+  } else {
+    const f32x4 got = *reinterpret_cast<const f32x4*>(p);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) x[e] = got[e];
+  }
+}
+
+template <class SI, class SO, int TAPS>
+__global__ __launch_bounds__(kThreads) void short_conv_run_kernel(
+    typename SO::T* __restrict__ out, int64_t out_stride, const typename SI::T* __restrict__ u,
+    int64_t u_stride, const float* __restrict__ w, const float* __restrict__ bias,
+    float* __restrict__ state, const int* __restrict__ query_start_loc,
+    const int* __restrict__ context_lens, const int* __restrict__ state_slots,
+    const int* __restrict__ token_seq, int num_tokens, int channels, int act, int run) {
+  constexpr int VC = 16 / sizeof(typename SI::T), B = TAPS - 1;
+  const int pieces = channels / VC;
+  const int64_t id = (int64_t)blockIdx.x * kThreads + threadIdx.x;
+  const int c = VC * (int)(id % pieces);
+  const int t0 = (int)(id / pieces) * run;
+  if (t0 >= num_tokens) return;
+  float wt[TAPS][VC], bs[VC];
+#pragma unroll
+  for (int v = 0; v < VC; ++v) {
+    bs[v] = bias != nullptr ? bias[c + v] : 0.f;
+#pragma unroll
+    for (int j = 0; j < TAPS; ++j) wt[j][v] = w[(int64_t)(c + v) * TAPS + j];
+  }
+  float before[B][VC];              // the inputs B, ..., 1 rows back
+  int b = -1;
+  const int t1 = min(t0 + run, num_tokens);
+  for (int t = t0; t < t1; ++t) {
+    if (token_seq[t] != b) {        // another sequence: its inputs ahead of this row
+      b = token_seq[t];
+      const int start = query_start_loc[b], ctx = context_lens[b];
+      const float* st = state + (int64_t)state_slots[b] * B * channels + c;
+#pragma unroll
+      for (int i = 0; i < B; ++i) {
+        const int back = B - i, row = t - back;
+        if (row >= start) {
+          load_channels<SI, VC>(u + (int64_t)row * u_stride + c, before[i]);
+        } else {
+          const int p = ctx + row - start;      // position; entry p - ctx + B of the old state
+#pragma unroll
+          for (int v = 0; v < VC; v += 4) {
+            f32x4 got = {0.f, 0.f, 0.f, 0.f};
+            if (p >= 0) got = *reinterpret_cast<const f32x4*>(st + (int64_t)(p - ctx + B) * channels + v);
+#pragma unroll
+            for (int e = 0; e < 4; ++e) before[i][v + e] = got[e];
+          }
+        }
+      }
+    }
+    float cur[VC], r[VC];
+    load_channels<SI, VC>(u + (int64_t)t * u_stride + c, cur);
+#pragma unroll
+    for (int v = 0; v < VC; ++v) {
+      float acc = bs[v];
+#pragma unroll
+      for (int i = 0; i < B; ++i) acc += wt[i][v] * before[i][v];
+      acc += wt[B][v] * cur[v];
+      if (sizeof(typename SO::T) == 2 && act == VLA_ACT_SILU)      // rounded to 16 bits right away
+        r[v] = acc * __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(-1.4426950408889634f * acc));
+      else
+        r[v] = activate(acc, act);
+    }
+    typename SO::T* o = out + (int64_t)t * out_stride + c;
+    if constexpr (sizeof(typename SO::T) == 2) {
+      uint32_t word[VC / 2];
+#pragma unroll
+      for (int e = 0; e < VC / 2; ++e) word[e] = pack16<SO>(r[2 * e], r[2 * e + 1]);
+      if constexpr (VC == 8)
+        *reinterpret_cast<u32x4*>(o) = u32x4{word[0], word[1], word[2], word[3]};
+      else
+        *reinterpret_cast<u32x2*>(o) = u32x2{word[0], word[1]};
+    } else {
+#pragma unroll
+      for (int v = 0; v < VC; v += 4) *reinterpret_cast<f32x4*>(o + v) = f32x4{r[v], r[v + 1], r[v + 2], r[v + 3]};
+    }
+#pragma unroll
+    for (int v = 0; v < VC; ++v) {
+#pragma unroll
+      for (int i = 0; i + 1 < B; ++i) before[i][v] = before[i + 1][v];
+      before[B - 1][v] = cur[v];
+    }
+    if (query_start_loc[b + 1] - query_start_loc[b] == 1) {
+      float* st = state + (int64_t)state_slots[b] * B * channels + c;
+#pragma unroll
+      for (int i = 0; i < B; ++i)
+#pragma unroll
+        for (int v = 0; v < VC; v += 4)
+          *reinterpret_cast<f32x4*>(st + (int64_t)i * channels + v) =
+              f32x4{before[i][v], before[i][v + 1], before[i][v + 2], before[i][v + 3]};
+    }
+  }
+}
+
 // The last taps - 1 inputs of every sequence of the step, oldest first.  A thread owns a channel:
-// it reads what it keeps of the old state before it writes.
+// it reads what it keeps of the old state before it writes.  skip_single: sequences with one row have
+// had their state written.
 template <class SI>
 __global__ __launch_bounds__(kThreads) void short_conv_state_kernel(
     float* __restrict__ state, const typename SI::T* __restrict__ u, int64_t u_stride,
     const int* __restrict__ query_start_loc, const int* __restrict__ context_lens,
-    const int* __restrict__ state_slots, int channels, int taps) {
+    const int* __restrict__ state_slots, int channels, int taps, bool skip_single) {
   const int b = blockIdx.y;
   const int c = blockIdx.x * kThreads + threadIdx.x;
   if (c >= channels) return;
   const int start = query_start_loc[b], n = query_start_loc[b + 1] - start, ctx = context_lens[b];
+  if (skip_single && n == 1) return;
   float* st = state + (int64_t)state_slots[b] * (taps - 1) * channels;
   float keep[kMaxTaps];
   for (int i = 0; i < taps - 1; ++i) {
@@ -219,7 +334,7 @@ extern "C" int vla_seq_short_conv(void* out, int64_t out_stride, int out_dtype, 
                                   const float* bias, float* state, const int* query_start_loc,
                                   const int* context_lens, const int* state_slots,
                                   const int* token_seq, int num_tokens, int num_seqs, int num_slots,
-                                  int channels, int taps, int act, void* stream) {
+                                  int channels, int taps, int act, int max_query_len, void* stream) {
   if (num_tokens == 0) return VLA_OK;
   if (!out || !u || !weight || !query_start_loc || !context_lens || !state_slots || !token_seq ||
       num_tokens < 0 || num_seqs <= 0 || num_seqs > 65535 || channels <= 0 || taps < 1 ||
@@ -229,19 +344,51 @@ extern "C" int vla_seq_short_conv(void* out, int64_t out_stride, int out_dtype, 
   return with_two(u_dtype, out_dtype, [&](auto si, auto so) {
     using SI = decltype(si);
     using SO = decltype(so);
-    short_conv_kernel<SI, SO><<<num_tokens, kThreads, 0, (hipStream_t)stream>>>(
-        (typename SO::T*)out, out_stride, (const typename SI::T*)u, u_stride, weight, bias, state,
-        query_start_loc, context_lens, state_slots, token_seq, channels, taps, act);
+    using TI = typename SI::T;
+    using TO = typename SO::T;
+    constexpr int VC = 16 / sizeof(TI);
+    const bool vec = taps >= 2 && taps <= 4 && channels % VC == 0 && ((uintptr_t)u % 16) == 0 &&
+                     u_stride % VC == 0 && (uintptr_t)out % (VC * sizeof(TO) < 16 ? VC * sizeof(TO) : 16) == 0 &&
+                     out_stride % VC == 0 && ((uintptr_t)state % 16) == 0 &&
+                     g_conv_kernel.load(std::memory_order_relaxed) == 0;
+    if (vec) {
+      const int run = num_tokens >= 1024 ? 8 : 1;
+      const int64_t threads = (int64_t)((num_tokens + run - 1) / run) * (channels / VC);
+      const unsigned blocks = (unsigned)((threads + kThreads - 1) / kThreads);
+      auto launch = [&](auto kernel) {
+        kernel<<<blocks, kThreads, 0, (hipStream_t)stream>>>((TO*)out, out_stride, (const TI*)u, u_stride, weight,
+                                                             bias, state, query_start_loc, context_lens,
+                                                             state_slots, token_seq, num_tokens, channels, act,
+                                                             run);
+      };
+      if (taps == 2)
+        launch(short_conv_run_kernel<SI, SO, 2>);
+      else if (taps == 3)
+        launch(short_conv_run_kernel<SI, SO, 3>);
+      else
+        launch(short_conv_run_kernel<SI, SO, 4>);
+    } else {
+      short_conv_kernel<SI, SO><<<num_tokens, kThreads, 0, (hipStream_t)stream>>>(
+          (TO*)out, out_stride, (const TI*)u, u_stride, weight, bias, state, query_start_loc, context_lens,
+          state_slots, token_seq, channels, taps, act);
+    }
     VLA_SEQ_HIP_CHECK(hipGetLastError());
-    if (taps > 1) {
+    if (taps > 1 && !(vec && max_query_len == 1)) {
       short_conv_state_kernel<SI><<<dim3((channels + kThreads - 1) / kThreads, num_seqs), kThreads, 0,
                                     (hipStream_t)stream>>>(state, (const typename SI::T*)u, u_stride,
                                                            query_start_loc, context_lens, state_slots,
-                                                           channels, taps);
+                                                           channels, taps, vec);
       VLA_SEQ_HIP_CHECK(hipGetLastError());
     }
     return VLA_OK;
   });
+}
+
+// 0: short_conv picks its kernel per shape; 1: always the one for any taps and alignment (tests run both)
+extern "C" int vla_seq_set_short_conv_kernel(int mode) {
+  if (mode < 0 || mode > 1) return VLA_ERR_ARG;
+  g_conv_kernel.store(mode, std::memory_order_relaxed);
+  return VLA_OK;
 }
 
 extern "C" int vla_seq_gated_act_lookup(void* out, int64_t out_stride, int out_dtype,
