@@ -330,14 +330,14 @@ int vla_seq_rms_norm_rows(void* out, int64_t out_stride, int out_dtype, const vo
  * sequence's start; weight fp32 [channels, taps], bias fp32 [channels] or null, act a VLA_ACT_*
  * code.  The last taps - 1 inputs of a sequence live in state fp32 [num_slots, taps - 1, channels]
  * (oldest first): rows of earlier steps are read from there, and the step leaves its own last
- * inputs there.  taps <= 32.  max_query_len: the longest run of the step (0: unknown).
+ * inputs there.  taps <= 32.
  * vla_seq_set_short_conv_kernel(1) keeps to the kernel for any taps and alignment (tests run both). */
 int vla_seq_set_short_conv_kernel(int mode);
 int vla_seq_short_conv(void* out, int64_t out_stride, int out_dtype, const void* u, int64_t u_stride,
                        int u_dtype, const float* weight, const float* bias, float* state,
                        const int* query_start_loc, const int* context_lens, const int* state_slots,
                        const int* token_seq, int num_tokens, int num_seqs, int num_slots,
-                       int channels, int taps, int act, int max_query_len, void* stream);
+                       int channels, int taps, int act, void* stream);
 
 /* out[t, c] = out_dtype(act(gate[t, c]) * table[ids[t], first_col + c]), c < features. */
 int vla_seq_gated_act_lookup(void* out, int64_t out_stride, int out_dtype, const void* gate,

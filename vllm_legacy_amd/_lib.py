@@ -129,7 +129,7 @@ def seq_lib():
         L.vla_seq_moe_route.argtypes = [p, i64, p, p, i64, p, p, p, p, p, p, i, i, i, i, i, i, i, p]
         L.vla_seq_post_norm.argtypes = [p, f, p, i64, i, p, f, p, i, i, i, p]
         L.vla_seq_rms_norm_rows.argtypes = [p, i64, i, p, i64, i, p, f, i, i, p]
-        L.vla_seq_short_conv.argtypes = [p, i64, i, p, i64, i, p, p, p, p, p, p, p, i, i, i, i, i, i, i, p]
+        L.vla_seq_short_conv.argtypes = [p, i64, i, p, i64, i, p, p, p, p, p, p, p, i, i, i, i, i, i, p]
         L.vla_seq_set_short_conv_kernel.argtypes = [i]
         L.vla_seq_gated_act_lookup.argtypes = [p, i64, i, p, i64, i, p, i64, i, p, i, i, i, i, i, p]
         L.vla_seq_embed_scaled.argtypes = [p, p, p, f, i, i, i, i, p]

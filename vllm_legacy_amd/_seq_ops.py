@@ -634,7 +634,7 @@ def rms_norm_rows(out: torch.Tensor, x: torch.Tensor, weight: torch.Tensor, eps:
 
 def short_conv(out: torch.Tensor, u: torch.Tensor, weight: torch.Tensor, bias: Optional[torch.Tensor],
                state: Optional[torch.Tensor], query_start_loc: torch.Tensor, context_lens: torch.Tensor,
-               state_slots: torch.Tensor, token_seq: torch.Tensor, act: str = "none", max_query_len: int = 0) -> None:
+               state_slots: torch.Tensor, token_seq: torch.Tensor, act: str = "none") -> None:
     """out = act(bias + conv(u)) along time per channel; out, u [T, C] views with free row strides;
     weight fp32 [C, taps]; state fp32 [slots, taps - 1, C] holds every sequence's last inputs and is
     brought up to date."""
@@ -658,7 +658,7 @@ def short_conv(out: torch.Tensor, u: torch.Tensor, weight: torch.Tensor, bias: O
             out.data_ptr(), _rows(out, Cn), _dt(out.dtype), u.data_ptr(), _rows(u, Cn), _dt(u.dtype),
             weight.data_ptr(), _p(bias), _p(state if taps > 1 else None), query_start_loc.data_ptr(),
             context_lens.data_ptr(), state_slots.data_ptr(), token_seq.data_ptr(), T, B, slots, Cn, taps, ACT[act],
-            int(max_query_len), _stream(u.device)), "short_conv")
+            _stream(u.device)), "short_conv")
 
 
 def set_short_conv_kernel(mode: int) -> None:

@@ -9,6 +9,7 @@
 //   softcap           z <- cap * tanh(z / cap)
 // One workgroup per row, fp32 arithmetic throughout; rows are read / written in the types named.
 #include <atomic>
+#include <type_traits>
 
 #include "seq_common.h"
 
@@ -119,84 +120,104 @@ __global__ __launch_bounds__(kThreads) void short_conv_kernel(
   }
 }
 
-// Two to four taps, rows and channels in whole 16-byte pieces: a thread takes 16 bytes of channels
-// through `run` consecutive rows of the step and keeps the taps - 1 inputs before the current row in
-// registers, so a row is read once per run and taps - 1 times more at its start.  Where a sequence
-// brings a single row (decode steps) the thread that has it also leaves the sequence's new state: no
-// other thread reads that slot.
+// Two to four taps, silu or no activation, rows and channels in whole 16-byte pieces: a thread takes 16 bytes of channels
+// through kRun consecutive rows of one sequence and keeps the taps - 1 inputs before the current row in
+// registers.  Runs are counted from a sequence's first row of the step (sequence b's are slots
+// start_b / kRun + b + 0, 1, ...), so only its first run needs the old state, and the thread that has it
+// leaves the new one: one launch, no thread reads what another writes.
+constexpr int kRun = 8;
+
 template <class S, int VC>
-__device__ __forceinline__ void load_channels(const typename S::T* p, float (&x)[VC]) {
+__device__ __forceinline__ void unpack_channels(u32x4 got, float (&x)[VC]) {
   if constexpr (sizeof(typename S::T) == 2) {
-    const u32x4 got = *reinterpret_cast<const u32x4*>(p);
 #pragma unroll
     for (int e = 0; e < 4; ++e) {
       x[2 * e] = lo16<S>(got[e]);
       x[2 * e + 1] = hi16<S>(got[e]);
     }
   } else {
-    const f32x4 got = *reinterpret_cast<const f32x4*>(p);
+    const f32x4 f = __builtin_bit_cast(f32x4, got);
 #pragma unroll
-    for (int e = 0; e < 4; ++e) x[e] = got[e];
+    for (int e = 0; e < 4; ++e) x[e] = f[e];
   }
 }
+template <class S, int VC>
+__device__ __forceinline__ void load_channels(const typename S::T* p, float (&x)[VC]) {
+  unpack_channels<S, VC>(*reinterpret_cast<const u32x4*>(p), x);
+}
 
-template <class SI, class SO, int TAPS>
+template <class SI, class SO, int TAPS, int ACT>
 __global__ __launch_bounds__(kThreads) void short_conv_run_kernel(
     typename SO::T* __restrict__ out, int64_t out_stride, const typename SI::T* __restrict__ u,
-    int64_t u_stride, const float* __restrict__ w, const float* __restrict__ bias,
-    float* __restrict__ state, const int* __restrict__ query_start_loc,
-    const int* __restrict__ context_lens, const int* __restrict__ state_slots,
-    const int* __restrict__ token_seq, int num_tokens, int channels, int act, int run) {
+    int64_t u_stride, const float* __restrict__ w, const float* __restrict__ bias, float* state,
+    const int* __restrict__ query_start_loc, const int* __restrict__ context_lens,
+    const int* __restrict__ state_slots, int num_seqs, int channels) {
   constexpr int VC = 16 / sizeof(typename SI::T), B = TAPS - 1;
-  const int pieces = channels / VC;
-  const int64_t id = (int64_t)blockIdx.x * kThreads + threadIdx.x;
-  const int c = VC * (int)(id % pieces);
-  const int t0 = (int)(id / pieces) * run;
-  if (t0 >= num_tokens) return;
+  const int c = VC * (blockIdx.x * blockDim.x + threadIdx.x);
+  if (c >= channels) return;
+  int lo = 0, hi = num_seqs - 1;                // the last sequence whose first slot is not behind this one
+  while (lo < hi) {
+    const int mid = (lo + hi + 1) >> 1;
+    if (query_start_loc[mid] / kRun + mid <= (int)blockIdx.y)
+      lo = mid;
+    else
+      hi = mid - 1;
+  }
+  const int start = query_start_loc[lo], end = query_start_loc[lo + 1];
+  const int run = blockIdx.y - (start / kRun + lo);
+  const int t0 = start + run * kRun, t1 = min(t0 + kRun, end);
+  if (t0 >= end) return;                        // a slot behind the sequence's last run
+  u32x4 rows[kRun];                             // the whole run is asked for before anything is used
+#pragma unroll
+  for (int i = 0; i < kRun; ++i)
+    rows[i] = *reinterpret_cast<const u32x4*>(u + (int64_t)min(t0 + i, t1 - 1) * u_stride + c);
   float wt[TAPS][VC], bs[VC];
 #pragma unroll
-  for (int v = 0; v < VC; ++v) {
-    bs[v] = bias != nullptr ? bias[c + v] : 0.f;
+  for (int i = 0; i < VC * TAPS; i += 4) {      // the weights of VC channels lie side by side
+    const f32x4 got = *reinterpret_cast<const f32x4*>(w + (int64_t)c * TAPS + i);
 #pragma unroll
-    for (int j = 0; j < TAPS; ++j) wt[j][v] = w[(int64_t)(c + v) * TAPS + j];
+    for (int e = 0; e < 4; ++e) wt[(i + e) % TAPS][(i + e) / TAPS] = got[e];
   }
-  float before[B][VC];              // the inputs B, ..., 1 rows back
-  int b = -1;
-  const int t1 = min(t0 + run, num_tokens);
-  for (int t = t0; t < t1; ++t) {
-    if (token_seq[t] != b) {        // another sequence: its inputs ahead of this row
-      b = token_seq[t];
-      const int start = query_start_loc[b], ctx = context_lens[b];
-      const float* st = state + (int64_t)state_slots[b] * B * channels + c;
 #pragma unroll
-      for (int i = 0; i < B; ++i) {
-        const int back = B - i, row = t - back;
-        if (row >= start) {
-          load_channels<SI, VC>(u + (int64_t)row * u_stride + c, before[i]);
-        } else {
-          const int p = ctx + row - start;      // position; entry p - ctx + B of the old state
+  for (int v = 0; v < VC; v += 4) {
+    f32x4 got = {0.f, 0.f, 0.f, 0.f};
+    if (bias != nullptr) got = *reinterpret_cast<const f32x4*>(bias + c + v);
 #pragma unroll
-          for (int v = 0; v < VC; v += 4) {
-            f32x4 got = {0.f, 0.f, 0.f, 0.f};
-            if (p >= 0) got = *reinterpret_cast<const f32x4*>(st + (int64_t)(p - ctx + B) * channels + v);
+    for (int e = 0; e < 4; ++e) bs[v + e] = got[e];
+  }
+  float before[B][VC];                          // the inputs B, ..., 1 rows back
+  const int ctx = context_lens[lo];
+  float* st = state + (int64_t)state_slots[lo] * B * channels + c;
 #pragma unroll
-            for (int e = 0; e < 4; ++e) before[i][v + e] = got[e];
-          }
-        }
+  for (int i = 0; i < B; ++i) {
+    if (run > 0) {
+      load_channels<SI, VC>(u + (int64_t)(t0 - B + i) * u_stride + c, before[i]);
+    } else {
+#pragma unroll
+      for (int v = 0; v < VC; v += 4) {         // entry i of the old state is position ctx - B + i
+        f32x4 got = {0.f, 0.f, 0.f, 0.f};
+        if (ctx - B + i >= 0) got = *reinterpret_cast<const f32x4*>(st + (int64_t)i * channels + v);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) before[i][v + e] = got[e];
       }
     }
+  }
+#pragma unroll
+  for (int k = 0; k < kRun; ++k) {
+    const int t = t0 + k;
+    if (t >= t1) break;
     float cur[VC], r[VC];
-    load_channels<SI, VC>(u + (int64_t)t * u_stride + c, cur);
+    unpack_channels<SI, VC>(rows[k], cur);
 #pragma unroll
     for (int v = 0; v < VC; ++v) {
       float acc = bs[v];
 #pragma unroll
       for (int i = 0; i < B; ++i) acc += wt[i][v] * before[i][v];
       acc += wt[B][v] * cur[v];
-      if (sizeof(typename SO::T) == 2 && act == VLA_ACT_SILU)      // rounded to 16 bits right away
+      if constexpr (ACT == VLA_ACT_SILU && sizeof(typename SO::T) == 2)      // rounded to 16 bits right away
         r[v] = acc * __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(-1.4426950408889634f * acc));
       else
-        r[v] = activate(acc, act);
+        r[v] = activate(acc, ACT);
     }
     typename SO::T* o = out + (int64_t)t * out_stride + c;
     if constexpr (sizeof(typename SO::T) == 2) {
@@ -217,31 +238,31 @@ __global__ __launch_bounds__(kThreads) void short_conv_run_kernel(
       for (int i = 0; i + 1 < B; ++i) before[i][v] = before[i + 1][v];
       before[B - 1][v] = cur[v];
     }
-    if (query_start_loc[b + 1] - query_start_loc[b] == 1) {
-      float* st = state + (int64_t)state_slots[b] * B * channels + c;
-#pragma unroll
-      for (int i = 0; i < B; ++i)
-#pragma unroll
-        for (int v = 0; v < VC; v += 4)
-          *reinterpret_cast<f32x4*>(st + (int64_t)i * channels + v) =
-              f32x4{before[i][v], before[i][v + 1], before[i][v + 2], before[i][v + 3]};
-    }
   }
+  if (run > 0) return;
+  if (t1 < end) {                               // the sequence goes on: its last inputs are other runs' rows
+#pragma unroll
+    for (int i = 0; i < B; ++i) load_channels<SI, VC>(u + (int64_t)(end - B + i) * u_stride + c, before[i]);
+  }
+#pragma unroll
+  for (int i = 0; i < B; ++i)
+#pragma unroll
+    for (int v = 0; v < VC; v += 4)
+      *reinterpret_cast<f32x4*>(st + (int64_t)i * channels + v) =
+          f32x4{before[i][v], before[i][v + 1], before[i][v + 2], before[i][v + 3]};
 }
 
 // The last taps - 1 inputs of every sequence of the step, oldest first.  A thread owns a channel:
-// it reads what it keeps of the old state before it writes.  skip_single: sequences with one row have
-// had their state written.
+// it reads what it keeps of the old state before it writes.
 template <class SI>
 __global__ __launch_bounds__(kThreads) void short_conv_state_kernel(
     float* __restrict__ state, const typename SI::T* __restrict__ u, int64_t u_stride,
     const int* __restrict__ query_start_loc, const int* __restrict__ context_lens,
-    const int* __restrict__ state_slots, int channels, int taps, bool skip_single) {
+    const int* __restrict__ state_slots, int channels, int taps) {
   const int b = blockIdx.y;
   const int c = blockIdx.x * kThreads + threadIdx.x;
   if (c >= channels) return;
   const int start = query_start_loc[b], n = query_start_loc[b + 1] - start, ctx = context_lens[b];
-  if (skip_single && n == 1) return;
   float* st = state + (int64_t)state_slots[b] * (taps - 1) * channels;
   float keep[kMaxTaps];
   for (int i = 0; i < taps - 1; ++i) {
@@ -334,7 +355,7 @@ extern "C" int vla_seq_short_conv(void* out, int64_t out_stride, int out_dtype, 
                                   const float* bias, float* state, const int* query_start_loc,
                                   const int* context_lens, const int* state_slots,
                                   const int* token_seq, int num_tokens, int num_seqs, int num_slots,
-                                  int channels, int taps, int act, int max_query_len, void* stream) {
+                                  int channels, int taps, int act, void* stream) {
   if (num_tokens == 0) return VLA_OK;
   if (!out || !u || !weight || !query_start_loc || !context_lens || !state_slots || !token_seq ||
       num_tokens < 0 || num_seqs <= 0 || num_seqs > 65535 || channels <= 0 || taps < 1 ||
@@ -347,37 +368,43 @@ extern "C" int vla_seq_short_conv(void* out, int64_t out_stride, int out_dtype, 
     using TI = typename SI::T;
     using TO = typename SO::T;
     constexpr int VC = 16 / sizeof(TI);
-    const bool vec = taps >= 2 && taps <= 4 && channels % VC == 0 && ((uintptr_t)u % 16) == 0 &&
+    const bool vec = taps >= 2 && taps <= 4 && (act == VLA_ACT_NONE || act == VLA_ACT_SILU) && channels % VC == 0 && ((uintptr_t)u % 16) == 0 &&
                      u_stride % VC == 0 && (uintptr_t)out % (VC * sizeof(TO) < 16 ? VC * sizeof(TO) : 16) == 0 &&
                      out_stride % VC == 0 && ((uintptr_t)state % 16) == 0 &&
-                     g_conv_kernel.load(std::memory_order_relaxed) == 0;
+                     ((uintptr_t)weight % 16) == 0 && ((uintptr_t)bias % 16) == 0 &&
+                     num_tokens / kRun + num_seqs <= 65535 && g_conv_kernel.load(std::memory_order_relaxed) == 0;
     if (vec) {
-      const int run = num_tokens >= 1024 ? 8 : 1;
-      const int64_t threads = (int64_t)((num_tokens + run - 1) / run) * (channels / VC);
-      const unsigned blocks = (unsigned)((threads + kThreads - 1) / kThreads);
+      const int pieces = channels / VC, blocks = (pieces + kThreads - 1) / kThreads;
+      const int threads = ((pieces + blocks - 1) / blocks + kWave - 1) / kWave * kWave;
+      const dim3 grid(blocks, num_tokens / kRun + num_seqs);
       auto launch = [&](auto kernel) {
-        kernel<<<blocks, kThreads, 0, (hipStream_t)stream>>>((TO*)out, out_stride, (const TI*)u, u_stride, weight,
-                                                             bias, state, query_start_loc, context_lens,
-                                                             state_slots, token_seq, num_tokens, channels, act,
-                                                             run);
+        kernel<<<grid, threads, 0, (hipStream_t)stream>>>((TO*)out, out_stride, (const TI*)u, u_stride, weight, bias,
+                                                          state, query_start_loc, context_lens, state_slots,
+                                                          num_seqs, channels);
+      };
+      auto by_act = [&](auto n) {
+        if (act == VLA_ACT_SILU)
+          launch(short_conv_run_kernel<SI, SO, decltype(n)::value, VLA_ACT_SILU>);
+        else
+          launch(short_conv_run_kernel<SI, SO, decltype(n)::value, VLA_ACT_NONE>);
       };
       if (taps == 2)
-        launch(short_conv_run_kernel<SI, SO, 2>);
+        by_act(std::integral_constant<int, 2>{});
       else if (taps == 3)
-        launch(short_conv_run_kernel<SI, SO, 3>);
+        by_act(std::integral_constant<int, 3>{});
       else
-        launch(short_conv_run_kernel<SI, SO, 4>);
+        by_act(std::integral_constant<int, 4>{});
     } else {
       short_conv_kernel<SI, SO><<<num_tokens, kThreads, 0, (hipStream_t)stream>>>(
           (TO*)out, out_stride, (const TI*)u, u_stride, weight, bias, state, query_start_loc, context_lens,
           state_slots, token_seq, channels, taps, act);
     }
     VLA_SEQ_HIP_CHECK(hipGetLastError());
-    if (taps > 1 && !(vec && max_query_len == 1)) {
+    if (taps > 1 && !vec) {
       short_conv_state_kernel<SI><<<dim3((channels + kThreads - 1) / kThreads, num_seqs), kThreads, 0,
                                     (hipStream_t)stream>>>(state, (const typename SI::T*)u, u_stride,
                                                            query_start_loc, context_lens, state_slots,
-                                                           channels, taps, vec);
+                                                           channels, taps);
       VLA_SEQ_HIP_CHECK(hipGetLastError());
     }
     return VLA_OK;

@@ -186,7 +186,7 @@ class ShortConv(nn.Module):
     def forward(self, out: torch.Tensor, u: torch.Tensor, state: Optional[torch.Tensor], batch) -> torch.Tensor:
         seq_ops.short_conv(out, u, self.weight.data, None if self.bias is None else self.bias.data,
                            state if self.taps > 1 else None, batch.query_start_loc, batch.context_lens,
-                           batch.state_slots, batch.token_seq, self.act, batch.max_query_len)
+                           batch.state_slots, batch.token_seq, self.act)
         return out
 
 
