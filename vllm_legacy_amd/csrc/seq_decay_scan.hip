@@ -83,10 +83,10 @@ __device__ __forceinline__ float load_one(const void* p, int64_t i, int dtype) {
   return ((const float*)p)[i];
 }
 
-// the log decay and the input's factor of row t
-__device__ __forceinline__ void row_decay(const DecayScan& a, int64_t t, int h, float& g, float& w) {
+// the log decay and the input's factor of a row (dt: its step size's projection, where there is one)
+__device__ __forceinline__ void row_decay(const DecayScan& a, float dt, int h, float& g, float& w) {
   if (a.dt != nullptr) {
-    w = softplus_f(load_one(a.dt, t * a.dt_stride + h, a.dtype) + a.dt_bias[h]);
+    w = softplus_f(dt + a.dt_bias[h]);
     g = -expf(a.a_log[h]) * w;
   } else {
     w = 1.f;
@@ -106,30 +106,30 @@ struct Piece<false> {
   f32x4 x, y;
 };
 
-// values first .. first + 7 of row `row` (null row: zeros), columns from `width` on are zeros
+// values first .. first + 7 of a row; with vec, width is a multiple of eight and a piece behind the row's
+// end reads its first piece instead (the reader of the pieces masks it), so that no load waits for
+// another's branch; otherwise columns from `width` on are zeros
 template <bool W16>
-__device__ __forceinline__ Piece<W16> read_piece(const void* base, int64_t at, int first, int width, bool row,
-                                                 bool vec) {
+__device__ __forceinline__ Piece<W16> read_piece(const void* base, int64_t at, int first, int width, bool vec) {
   Piece<W16> p;
+  if (vec) first = first < width ? first : 0;
   if constexpr (W16) {
-    p.x = u32x4{0u, 0u, 0u, 0u};
-    if (!row || first >= width) return p;
     const uint16_t* src = (const uint16_t*)base + at + first;
     if (vec) {
       p.x = *reinterpret_cast<const u32x4*>(src);
     } else {
+      p.x = u32x4{0u, 0u, 0u, 0u};
 #pragma unroll
       for (int e = 0; e < 8; ++e)
         if (first + e < width) p.x[e >> 1] |= (uint32_t)src[e] << (16 * (e & 1));
     }
   } else {
-    p.x = p.y = f32x4{0.f, 0.f, 0.f, 0.f};
-    if (!row || first >= width) return p;
     const float* src = (const float*)base + at + first;
     if (vec) {
       p.x = *reinterpret_cast<const f32x4*>(src);
       p.y = *reinterpret_cast<const f32x4*>(src + 4);
     } else {
+      p.x = p.y = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
       for (int e = 0; e < 4; ++e) {
         if (first + e < width) p.x[e] = src[e];
@@ -138,6 +138,19 @@ __device__ __forceinline__ Piece<W16> read_piece(const void* base, int64_t at, i
     }
   }
   return p;
+}
+
+template <bool W16>
+__device__ __forceinline__ void mask_piece(Piece<W16>& p, bool live) {
+#pragma unroll
+  for (int e = 0; e < 4; ++e) {
+    if constexpr (W16) {
+      p.x[e] = live ? p.x[e] : 0u;
+    } else {
+      p.x[e] = live ? p.x[e] : 0.f;
+      p.y[e] = live ? p.y[e] : 0.f;
+    }
+  }
 }
 
 // a piece's values in fp32 after the activation, to LDS (16-byte aligned)
@@ -264,35 +277,35 @@ __global__ __launch_bounds__(64 * WAVES) void decay_block_kernel(DecayScan a) {
   double log_total = 0.0;
 
   Piece<W16> pq[NQ], pk[NQ], pv[NVP];
-  float row_g = 0.f, row_w = 0.f;
+  float row_dt = 0.f;
   auto fetch = [&](int t0) {
     const int n = min(kBlock, t_end - t0);
 #pragma unroll
     for (int u = 0; u < NQ; ++u) {
       const int i = tid + THREADS * u, r = i / (DP / 8), d = 8 * (i % (DP / 8));
-      const bool row = r < n;
-      pk[u] = read_piece<W16>(a.k, (int64_t)(t0 + r) * a.k_stride + (int64_t)hg * D, d, D, row, a.vec_k);
-      if (!STATE_ONLY)
-        pq[u] = read_piece<W16>(a.q, (int64_t)(t0 + r) * a.q_stride + (int64_t)hg * D, d, D, row, a.vec_q);
+      const int64_t t = t0 + min(r, n - 1);
+      pk[u] = read_piece<W16>(a.k, t * a.k_stride + (int64_t)hg * D, d, D, a.vec_k);
+      if (!STATE_ONLY) pq[u] = read_piece<W16>(a.q, t * a.q_stride + (int64_t)hg * D, d, D, a.vec_q);
     }
 #pragma unroll
     for (int u = 0; u < NVP; ++u) {
       const int i = tid + THREADS * u, r = i / (VB / 8), d = v0 + 8 * (i % (VB / 8));
-      pv[u] = read_piece<W16>(a.v, (int64_t)(t0 + r) * a.v_stride + (int64_t)h * V, d, V, r < n, a.vec_v);
+      pv[u] = read_piece<W16>(a.v, (int64_t)(t0 + min(r, n - 1)) * a.v_stride + (int64_t)h * V, d, V, a.vec_v);
     }
-    if (tid < kBlock) {
-      row_g = row_w = 0.f;
-      if (tid < n) row_decay(a, t0 + tid, h, row_g, row_w);
-    }
+    if (tid < kBlock && a.dt != nullptr)
+      row_dt = load_one(a.dt, (int64_t)(t0 + min(tid, n - 1)) * a.dt_stride + h, a.dtype);
   };
-  auto land_qk = [&](E* dst, const Piece<W16>& p) {
+  auto land_qk = [&](E* dst, Piece<W16>& p, bool live) {
+    mask_piece<W16>(p, live);
     if constexpr (QK16)
       *reinterpret_cast<u32x4*>(dst) = p.x;
     else
       land_piece<W16>(dst, p, a.act, a.dtype);
   };
-  auto land = [&]() {
+  auto land = [&](int n) {
     if (w == 0) {
+      float row_g = 0.f, row_w = 0.f;
+      if (lane < n) row_decay(a, row_dt, h, row_g, row_w);
       double cs = row_g;                                // inclusive sum over the 64 rows
 #pragma unroll
       for (int m = 1; m < 64; m <<= 1) {
@@ -310,12 +323,13 @@ __global__ __launch_bounds__(64 * WAVES) void decay_block_kernel(DecayScan a) {
     for (int u = 0; u < NQ; ++u) {
       const int i = tid + THREADS * u, r = i / (DP / 8), d = 8 * (i % (DP / 8));
       if (DP * kBlock / 8 % THREADS != 0 && r >= kBlock) continue;
-      land_qk(k_lds + r * KR + d, pk[u]);
-      if (!STATE_ONLY) land_qk(q_lds + r * KR + d, pq[u]);
+      land_qk(k_lds + r * KR + d, pk[u], r < n && d < D);
+      if (!STATE_ONLY) land_qk(q_lds + r * KR + d, pq[u], r < n && d < D);
     }
 #pragma unroll
     for (int u = 0; u < NVP; ++u) {
       const int i = tid + THREADS * u, r = i / (VB / 8), d = 8 * (i % (VB / 8));
+      mask_piece<W16>(pv[u], r < n && v0 + d < V);
       land_piece<W16>(v_lds + r * VR + d, pv[u], a.act, a.dtype);
     }
   };
@@ -339,7 +353,7 @@ __global__ __launch_bounds__(64 * WAVES) void decay_block_kernel(DecayScan a) {
   fetch(t_begin);
   for (int t0 = t_begin; t0 < t_end; t0 += kBlock) {
     const int n = min(kBlock, t_end - t0);
-    land();
+    land(n);
     __syncthreads();
     if (t0 + kBlock < t_end) fetch(t0 + kBlock);
     if constexpr (!STATE_ONLY) {
@@ -507,7 +521,7 @@ __global__ __launch_bounds__(256) void decay_step_kernel(DecayScan a) {
   };
   for (int t = t_begin; t < t_end; ++t) {
     float g, wt;
-    row_decay(a, t, h, g, wt);
+    row_decay(a, a.dt != nullptr ? load_one(a.dt, (int64_t)t * a.dt_stride + h, a.dtype) : 0.f, h, g, wt);
     const float e = expf(g);
     for (int d = tid; d < D; d += 256) {
       q_lds[d] = load(a.q, (int64_t)t * a.q_stride + (int64_t)hg * D + d);
@@ -787,8 +801,7 @@ extern "C" int vla_seq_decay_scan(float* o, const void* q, int64_t q_stride, con
     a.piece_decay = scratch + slots * heads * ((int64_t)dim * vdim);
     pieces = (int)slots;
   }
-  // Runs of a few rows first: in a mixed step both launches skip the other's sequences.  With one run per
-  // sequence and no more rows than the sequences could have in short runs there may be both kinds.
+  // a step of several sequences may hold runs of both kinds: each launch skips the other's sequences
   const bool steps = a.mode == 1 || (a.mode == 0 && (max_query_len <= kStepRows || num_seqs > 1));
   const bool blocks = a.mode == 2 || (a.mode == 0 && max_query_len > kStepRows);
   if (steps) {
