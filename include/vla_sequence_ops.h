@@ -151,6 +151,18 @@ int vla_seq_residual_norms(float* x, const void* y, int64_t y_stride, int y_dtyp
                            int num_tokens, int width, int out_dtype, float y_scale, const void* y2,
                            int64_t y2_stride, const float* post_weight2, void* stream);
 
+/* The stream's update of a layer whose branches all read the stream of its start:
+ *   x += s0 y0 + s1 y1 + s2 y2 + sum_k pair_weight[t, k] expert_rows[pair_row[t, k]]
+ * then out0 = x / sqrt(mean(x^2) + eps) * weight0 and out1 with weight1 (`out_dtype`).  Every part may
+ * be null (y1, y2 only with y0, out1 only with out0); y fp32 [T, width], expert_rows fp32 [rows,
+ * width], pair_row int32 (negative: nothing) and pair_weight fp32 [T, top], weights fp32 [width]; all
+ * contiguous. */
+int vla_seq_branch_sum_norms(float* x, const float* y0, float s0, const float* y1, float s1,
+                             const float* y2, float s2, const float* expert_rows,
+                             const int* pair_row, const float* pair_weight, int top, void* out0,
+                             const float* weight0, void* out1, const float* weight1, float eps,
+                             int num_tokens, int width, int out_dtype, void* stream);
+
 /* Causal convolution over time on each channel, added to its input:
  *   out[t] = dtype(h[t] + sum_j weight[:, j] h[t - taps + 1 + j]),  zeros before a sequence's start,
  * h fp32 [T, width], weight fp32 [width, taps].  The last taps - 1 inputs of a sequence live in
@@ -272,14 +284,17 @@ int vla_seq_mingru_scan(void* out, int64_t out_stride, const void* zp, int64_t z
  * softmax over the chosen logits), their s as they are without.  experts int32 / weights fp32 [T, top].  shared_gate given:
  * shared_gate[t] = sigmoid(shared_gate_weight . h), shared_gate_weight fp32 [width].  logits given
  * (fp32 rows of routed (+ 1 with a shared gate, its logit last) values, stride logits_stride): the
- * products are the caller's and h, router, shared_gate_weight are not read. */
+ * products are the caller's and h, router, shared_gate_weight are not read.  The experts form `groups`
+ * equal groups of neighbours; only those of the keep_groups groups whose largest s + correction is
+ * largest can be chosen (1 and 1: all).  Every weight leaves times weight_scale. */
 #define VLA_SCORE_SOFTMAX 0
 #define VLA_SCORE_SIGMOID 1
 int vla_seq_moe_route(const void* h, int64_t h_stride, const float* router, const float* logits,
                       int64_t logits_stride, const float* bias, const float* correction,
                       const float* shared_gate_weight, int* experts, float* weights,
                       float* shared_gate, int num_tokens, int width, int routed, int top, int score,
-                      int renormalize, int dtype, void* stream);
+                      int renormalize, int groups, int keep_groups, float weight_scale, int dtype,
+                      void* stream);
 
 /* Groups the pairs (token, choice) whose expert is below num_experts by expert, every group padded
  * to whole tiles of vla_seq_moe_tile_rows() rows: pair_row int32 [T * top] (-1: the pair's expert
@@ -378,14 +393,42 @@ int vla_seq_delta_rule_scan(void* out, int64_t out_stride, int out_dtype, const 
                             int num_seqs, int max_query_len, int num_slots, int heads, int kv_heads,
                             int dim, int vdim, float eps, float* scratch, void* stream);
 
+/* The delta rule with a decay per key channel: per head, on a state S fp32 [dim, vdim] (stored
+ * [num_slots, heads, vdim, dim]):
+ *   S <- diag(g) S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q
+ * k, q as above (unit vectors of the head's key head, q also times dim^-1/2), beta = sigmoid(beta row),
+ * g = exp(-exp(a_log[head]) softplus(z row + dt_bias)) per head and channel.  q, k [T, kv_heads * dim],
+ * v [T, heads * vdim], beta [T, heads]: `dtype` rows with their own strides; z fp32 [T, heads * dim];
+ * dt_bias fp32 [heads * dim], a_log fp32 [heads]; o fp32 [T, heads * vdim] contiguous.  A sequence
+ * with context 0 starts from zero.  scratch (fp32, vla_seq_channel_delta_scratch_floats values,
+ * 16-byte aligned) holds what the 16-row blocks of longer runs prepare.  max_query_len: the longest run
+ * of the step.  dim up to 1024 (above 256 every run goes token by token). */
+int64_t vla_seq_channel_delta_scratch_floats(int num_tokens, int num_seqs, int max_query_len, int heads,
+                                             int dim, int vdim);
+int vla_seq_channel_delta_scan(float* o, const void* q, int64_t q_stride, const void* k,
+                               int64_t k_stride, const void* v, int64_t v_stride, const void* beta,
+                               int64_t beta_stride, const float* z, int64_t z_stride,
+                               const float* dt_bias, const float* a_log, float* state,
+                               const int* query_start_loc, const int* context_lens,
+                               const int* state_slots, int num_tokens, int num_seqs, int num_slots,
+                               int max_query_len, int heads, int kv_heads, int dim, int vdim,
+                               float* scratch, int64_t scratch_floats, int dtype, void* stream);
+/* Kernel choice for tests: 0 = per run of rows (at most four token by token, longer ones in blocks),
+ * 1 = always token by token, 2 = always in blocks. */
+int vla_seq_set_channel_delta_kernel(int mode);
+
 /* ---- linear recurrence with one decay per head and token -------------------------------------------- */
 
 /* Per head, on a state S [dim, vdim] in fp32:
  *   S <- e^g S + w k v^T;   o = S^T q + skip v
  * with q, k of the head's group (heads / groups heads share one query / key) and either
  *   dt given:  w = softplus(dt row + dt_bias), g = -exp(a_log) w   (a state-space layer), or
- *   dt null:   w = 1, g = log_decay[head]                          (constant decays).
- * q, k and v pass `act` (VLA_ACT_NONE or VLA_ACT_SILU) first.  q, k [T, groups * dim],
+ *   row_log given: g = row_log[t, head] <= 0, w = row_weight[t, head] (fp32 [T, heads]), or
+ *   neither:   w = 1, g = log_decay[head]                          (constant decays).
+ * q, k and v pass `act` (VLA_ACT_NONE or VLA_ACT_SILU) first; q is multiplied by q_scale.
+ * norm_scale given (fp32 [T, heads], written): a normalizer n <- e^g n + w k runs beside S and
+ * norm_scale = 1 / (max(|n . q|, row_floor[t, head]) + norm_eps); a head's state is then dim * vdim
+ * numbers of S followed by dim of n (fp32 [num_slots, heads, dim * (vdim + 1)]).  q, k [T, groups * dim],
  * v [T, heads * vdim], dt [T, heads]: `dtype` rows with their own strides; dt_bias, a_log, log_decay,
  * skip (null: none) fp32 [heads]; o fp32 [T, heads * vdim] contiguous; state fp32 [num_slots, heads,
  * dim, vdim]; a sequence with context 0 starts from zero whatever its slot held.  Runs of more than
@@ -394,11 +437,13 @@ int vla_seq_delta_rule_scan(void* out, int64_t out_stride, int out_dtype, const 
  * the step. */
 #define VLA_DECAY_SCAN_PIECE 256
 int64_t vla_seq_decay_scan_scratch_floats(int num_tokens, int num_seqs, int max_query_len, int heads,
-                                          int dim, int vdim);
+                                          int dim, int vdim, int normalizer);
 int vla_seq_decay_scan(float* o, const void* q, int64_t q_stride, const void* k, int64_t k_stride,
                        const void* v, int64_t v_stride, const void* dt, int64_t dt_stride,
                        const float* dt_bias, const float* a_log, const float* log_decay,
-                       const float* skip, float* state, const int* query_start_loc,
+                       const float* skip, const float* row_log, const float* row_weight,
+                       const float* row_floor, float* norm_scale, float norm_eps, float q_scale,
+                       float* state, const int* query_start_loc,
                        const int* context_lens, const int* state_slots, int num_tokens, int num_seqs,
                        int num_slots, int max_query_len, int heads, int groups, int dim, int vdim,
                        int act, float* scratch, int64_t scratch_floats, int dtype, void* stream);
@@ -406,16 +451,31 @@ int vla_seq_decay_scan(float* o, const void* q, int64_t q_stride, const void* k,
  * blocks on the matrix cores), 1 = always token by token, 2 = always in blocks. */
 int vla_seq_set_decay_scan_kernel(int mode);
 
+/* Gates of a matrix memory with a running maximum, per (token, head):
+ *   i = cap tanh((zi + bias_i) / cap),  f = -softplus(-cap tanh((zf + bias_f) / cap)),
+ *   m_t = max(f + m_(t-1), i)  (0 before a sequence's start),
+ *   row_log = f + m_(t-1) - m_t,  row_weight = e^(i - m_t),  row_floor = e^(-m_t)
+ * zi, zf `dtype` [T, heads] with their own row strides, biases fp32 [heads], outputs fp32 [T, heads],
+ * maximum fp32 [num_slots, heads] (a sequence with context 0 starts from 0). */
+int vla_seq_matrix_memory_gates(float* row_log, float* row_weight, float* row_floor, const void* zi,
+                                int64_t zi_stride, const void* zf, int64_t zf_stride,
+                                const float* bias_i, const float* bias_f, float cap, float* maximum,
+                                const int* query_start_loc, const int* context_lens,
+                                const int* state_slots, int num_seqs, int num_slots,
+                                int max_query_len, int heads, int dtype, void* stream);
+
 /* A recurrence's output rows o [T, n] (fp32, contiguous), gated and normed in `groups` equal parts
  * (each by its own root mean square, eps inside the root):
  *   gate_first:  u = o * gate_act(gate);  out = u / rms(u) * weight
  *   otherwise:   out = o / rms(o) * weight * gate_act(gate)
- * weight fp32 [n]; gate and out `dtype` rows of n values with their own strides. */
+ * weight fp32 [n]; gate and out `dtype` rows of n values with their own strides; part_scale (null:
+ * none; fp32 [T, groups]) multiplies every part of o first. */
 #define VLA_GATE_SILU 0
 #define VLA_GATE_SIGMOID 1
 int vla_seq_gated_group_rms_norm(void* out, int64_t out_stride, const float* o, const float* weight,
                                  const void* gate, int64_t gate_stride, int gate_act, int gate_first,
-                                 int groups, float eps, int num_tokens, int n, int dtype, void* stream);
+                                 int groups, float eps, int num_tokens, int n, int dtype,
+                                 const float* part_scale, void* stream);
 
 /* ---- real-gated linear recurrent unit ------------------------------------------------------------- */
 
@@ -455,7 +515,8 @@ int vla_seq_latent_rotary_write(void* q, int64_t q_stride, int q_head_stride, in
  * of (q_lat[t, h] . c_j + q_rot[t, h] . k_rot_j) * scale; q_lat, q_rot and out are addressed by a
  * token stride and a head stride each.  window > 0 keeps the keys with position - j < window only;
  * gate (null: none; one number per (token, head), row stride gate_stride) multiplies a head's sums
- * by its sigmoid.  Any dtype, rank and rot up to 1024. */
+ * by its sigmoid; sinks (null: none; fp32 [heads]) adds exp(sink) to a head's softmax denominator, a
+ * key without a value whose score is not scaled.  Any dtype, rank and rot up to 1024. */
 int vla_seq_latent_attention(void* out, int64_t out_token_stride, int64_t out_head_stride,
                              const void* q_lat, int64_t lat_token_stride, int64_t lat_head_stride,
                              const void* q_rot, int64_t rot_token_stride, int64_t rot_head_stride,
@@ -463,7 +524,7 @@ int vla_seq_latent_attention(void* out, int64_t out_token_stride, int64_t out_he
                              const int* token_seq, const int64_t* positions, int num_tokens,
                              int heads, int rank, int rot, int block_size, int num_blocks,
                              float scale, int dtype, int window, const void* gate,
-                             int64_t gate_stride, void* stream);
+                             int64_t gate_stride, const float* sinks, void* stream);
 
 /* The same attention on the matrix cores for 16-bit models: 32 query rows that are (token, head)
  * pairs of one sequence per workgroup, tiles of 32 keys.  rank a multiple of 32 up to 512, rot a
@@ -484,7 +545,8 @@ int vla_seq_latent_attention_tiles(void* out, int64_t out_token_stride, int64_t 
                                    int num_seqs, int max_query_len, int heads, int rank, int rot,
                                    int block_size, int num_blocks, float scale, int key_splits,
                                    float* scratch, int num_tokens, int dtype, int window,
-                                   const void* gate, int64_t gate_stride, void* stream);
+                                   const void* gate, int64_t gate_stride, const float* sinks,
+                                   void* stream);
 int vla_seq_set_latent_attention_kernel(int mode);
 
 /* Kernel choice for tests: window attention 0 = per shape, 1 = one wave per (row, head);

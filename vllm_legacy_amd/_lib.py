@@ -66,7 +66,9 @@ SEQ_EXPORTS = [
     "vla_seq_latent_attention_tiles_supported", "vla_seq_latent_attention_scratch_floats", "vla_seq_set_latent_attention_kernel",
     "vla_seq_clamped_glu", "vla_seq_pair_hash_embed",
     "vla_seq_decay_scan", "vla_seq_decay_scan_scratch_floats", "vla_seq_set_decay_scan_kernel",
-    "vla_seq_gated_group_rms_norm", "vla_seq_set_short_conv_kernel",
+    "vla_seq_gated_group_rms_norm", "vla_seq_set_short_conv_kernel", "vla_seq_matrix_memory_gates",
+    "vla_seq_channel_delta_scan", "vla_seq_channel_delta_scratch_floats", "vla_seq_set_channel_delta_kernel",
+    "vla_seq_branch_sum_norms",
 ]
 _seq_lib = None
 
@@ -126,7 +128,7 @@ def seq_lib():
         L.vla_seq_mingru_scratch_floats.restype = i64
         L.vla_seq_mingru_scan.argtypes = [p, i64, p, i64, p, i64, p, i64, p, p, p, p, i, i, i, i, p,
                                           i64, i, p]
-        L.vla_seq_moe_route.argtypes = [p, i64, p, p, i64, p, p, p, p, p, p, i, i, i, i, i, i, i, p]
+        L.vla_seq_moe_route.argtypes = [p, i64, p, p, i64, p, p, p, p, p, p, i, i, i, i, i, i, i, i, f, i, p]
         L.vla_seq_post_norm.argtypes = [p, f, p, i64, i, p, f, p, i, i, i, p]
         L.vla_seq_rms_norm_rows.argtypes = [p, i64, i, p, i64, i, p, f, i, i, p]
         L.vla_seq_short_conv.argtypes = [p, i64, i, p, i64, i, p, p, p, p, p, p, p, i, i, i, i, i, i, p]
@@ -144,25 +146,32 @@ def seq_lib():
         L.vla_seq_latent_rotary_write.argtypes = [p, i64, i, i, p, i64, p, f, p, p, p, p, f, i, i, i, i, i,
                                                   i, i, i, i, p]
         L.vla_seq_latent_attention.argtypes = [p, i64, i64, p, i64, i64, p, i64, i64, p, p, i, p, p, i, i,
-                                               i, i, i, i, f, i, i, p, i64, p]
+                                               i, i, i, i, f, i, i, p, i64, p, p]
         L.vla_seq_moe_tile_rows.argtypes = []
         L.vla_seq_moe_plan.argtypes = [p, i, i, i, p, p, p, i, p, p, p]
         L.vla_seq_grouped_linear.argtypes = [p, i64, i, p, i64, p, p, p, i, i, i, i, p, i, p]
         L.vla_seq_moe_combine.argtypes = [p, p, p, p, p, i64, p, p, i, i, i, i, p]
         L.vla_seq_latent_attention_tiles_supported.argtypes = [i, i, i]
         L.vla_seq_latent_attention_tiles.argtypes = [p, i64, i64, p, i64, i64, p, i64, i64, p, p, i, p, p, i, i,
-                                                     i, i, i, i, i, f, i, p, i, i, i, p, i64, p]
+                                                     i, i, i, i, i, f, i, p, i, i, i, p, i64, p, p]
         L.vla_seq_clamped_glu.argtypes = [p, i64, p, i64, p, i64, i, i, f, f, f, i, p]
         L.vla_seq_pair_hash_embed.argtypes = [p, p, p, p, p, p, p, p, p, i, i, i, i, i, i64, i64, i64, i, p]
         L.vla_seq_latent_attention_scratch_floats.argtypes = [i, i, i, i]
         L.vla_seq_latent_attention_scratch_floats.restype = i64
         L.vla_seq_set_latent_attention_kernel.argtypes = [i]
-        L.vla_seq_decay_scan.argtypes = [p, p, i64, p, i64, p, i64, p, i64, p, p, p, p, p, p, p, p, i, i, i, i,
-                                         i, i, i, i, i, p, i64, i, p]
-        L.vla_seq_decay_scan_scratch_floats.argtypes = [i, i, i, i, i, i]
+        L.vla_seq_decay_scan.argtypes = [p, p, i64, p, i64, p, i64, p, i64, p, p, p, p, p, p, p, p, f, f, p, p, p, p,
+                                         i, i, i, i, i, i, i, i, i, p, i64, i, p]
+        L.vla_seq_decay_scan_scratch_floats.argtypes = [i, i, i, i, i, i, i]
         L.vla_seq_decay_scan_scratch_floats.restype = i64
         L.vla_seq_set_decay_scan_kernel.argtypes = [i]
-        L.vla_seq_gated_group_rms_norm.argtypes = [p, i64, p, p, p, i64, i, i, i, f, i, i, i, p]
+        L.vla_seq_gated_group_rms_norm.argtypes = [p, i64, p, p, p, i64, i, i, i, f, i, i, i, p, p]
+        L.vla_seq_matrix_memory_gates.argtypes = [p, p, p, p, i64, p, i64, p, p, f, p, p, p, p, i, i, i, i, i, p]
+        L.vla_seq_channel_delta_scan.argtypes = [p, p, i64, p, i64, p, i64, p, i64, p, i64, p, p, p, p, p, p, i, i, i,
+                                                 i, i, i, i, i, p, i64, i, p]
+        L.vla_seq_channel_delta_scratch_floats.argtypes = [i, i, i, i, i, i]
+        L.vla_seq_channel_delta_scratch_floats.restype = i64
+        L.vla_seq_set_channel_delta_kernel.argtypes = [i]
+        L.vla_seq_branch_sum_norms.argtypes = [p, p, f, p, f, p, f, p, p, p, i, p, p, p, p, f, i, i, i, p]
         _seq_lib = L
     return _seq_lib
 

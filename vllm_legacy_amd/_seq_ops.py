@@ -292,6 +292,34 @@ def residual_norms(x: torch.Tensor, y: Optional[torch.Tensor] = None, y_bias: Op
             _p(post_weight2), _stream(x.device)), "residual_norms")
 
 
+def branch_sum_norms(x: torch.Tensor, terms=(), experts=None, outs=(), eps: float = 1e-5) -> None:
+    """x (fp32 [T, W], in place) += the sum of up to three terms (y fp32 [T, W], factor) and, with experts =
+    (y fp32 [rows, W], pair_row int32 [T, top], weights fp32 [T, top]), of a token's expert rows; then for
+    each of up to two (out, weight): out = x / rms(x) * weight."""
+    T, W = x.shape
+    terms, outs = [(y, float(f)) for y, f in terms], list(outs)
+    assert x.dtype == torch.float32 and x.is_contiguous() and len(terms) <= 3 and len(outs) <= 2
+    _gpu(x, *[y for y, _ in terms], *(experts or ()), *[t for pair in outs for t in pair])
+    for y, _ in terms:
+        assert y.dtype == torch.float32 and y.is_contiguous() and y.shape == (T, W)
+    for out, w in outs:
+        assert out.shape == (T, W) and out.is_contiguous() and out.dtype == outs[0][0].dtype
+        assert w.dtype == torch.float32 and w.is_contiguous() and w.numel() == W
+    rows, pair_row, weights = experts or (None, None, None)
+    if experts is not None:
+        assert rows.dtype == torch.float32 and rows.is_contiguous() and rows.shape[1] == W
+        assert pair_row.dtype == torch.int32 and pair_row.is_contiguous() and pair_row.shape[0] == T
+        assert weights.dtype == torch.float32 and weights.is_contiguous() and weights.shape == pair_row.shape
+    terms += [(None, 0.0)] * (3 - len(terms))
+    dt = _lib.F32 if not outs else _dt(outs[0][0].dtype)
+    outs += [(None, None)] * (2 - len(outs))
+    with torch.cuda.device(x.device):
+        seq_check(_lib.seq_lib().vla_seq_branch_sum_norms(
+            x.data_ptr(), *[v for y, f in terms for v in (_p(y), f)], _p(rows), _p(pair_row), _p(weights),
+            0 if pair_row is None else pair_row.shape[1], *[_p(t) for pair in outs for t in pair], float(eps), T, W, dt,
+            _stream(x.device)), "branch_sum_norms")
+
+
 def causal_conv(out: torch.Tensor, h: torch.Tensor, weight: torch.Tensor, state: Optional[torch.Tensor],
                 query_start_loc: torch.Tensor, context_lens: torch.Tensor, state_slots: torch.Tensor,
                 token_seq: torch.Tensor) -> None:
@@ -516,11 +544,14 @@ def mingru_scan(out: torch.Tensor, zp: torch.Tensor, up: torch.Tensor, gp: torch
 
 def moe_route(h: torch.Tensor, router: torch.Tensor, correction: Optional[torch.Tensor],
               shared_gate_weight: Optional[torch.Tensor], top: int, logits: Optional[torch.Tensor] = None,
-              bias: Optional[torch.Tensor] = None, score: str = "softmax", renormalize: bool = True):
+              bias: Optional[torch.Tensor] = None, score: str = "softmax", renormalize: bool = True,
+              groups: int = 1, keep_groups: int = 1, weight_scale: float = 1.0):
     """-> experts int32 [T, top], weights fp32 [T, top], shared gate fp32 [T] or None.  logits
     (fp32 [T, routed (+ 1, the shared gate's last)]): the router products, when the caller formed
     them as one matrix product.  score: "softmax" over all experts or "sigmoid" of each logit; renormalize:
-    the chosen scores are divided by their sum."""
+    the chosen scores are divided by their sum; only experts of the keep_groups best of `groups` equal
+    groups of neighbours (a group counts as its best expert) can be chosen; weights leave times
+    weight_scale."""
     _gpu(h, router, correction, shared_gate_weight, logits, bias)
     T, W = h.shape
     N = router.shape[0]
@@ -538,7 +569,8 @@ def moe_route(h: torch.Tensor, router: torch.Tensor, correction: Optional[torch.
         seq_check(_lib.seq_lib().vla_seq_moe_route(
             h.data_ptr(), _rows(h, W), router.data_ptr(), _p(logits), 0 if logits is None else logits.shape[1],
             _p(bias), _p(correction), _p(shared_gate_weight), experts.data_ptr(), weights.data_ptr(), _p(sg), T, W, N,
-            int(top), MOE_SCORE[score], int(bool(renormalize)), _dt(h.dtype), _stream(h.device)), "moe_route")
+            int(top), MOE_SCORE[score], int(bool(renormalize)), int(groups), int(keep_groups), float(weight_scale),
+            _dt(h.dtype), _stream(h.device)), "moe_route")
     return experts, weights, sg
 
 
@@ -737,36 +769,87 @@ def set_delta_kernel(mode: int) -> None:
     seq_check(_lib.seq_lib().vla_seq_set_delta_kernel(mode), "set_delta_kernel")
 
 
+def channel_delta_scan(o: torch.Tensor, q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, beta: torch.Tensor,
+                       z: torch.Tensor, dt_bias: torch.Tensor, a_log: torch.Tensor, state: torch.Tensor,
+                       query_start_loc: torch.Tensor, context_lens: torch.Tensor, state_slots: torch.Tensor,
+                       kv_heads: int, max_query_len: int) -> None:
+    """Delta rule with a decay exp(-exp(a_log[h]) softplus(z + dt_bias)) per head and channel.  o fp32
+    [T, H*V]; q, k [T, G*D], v [T, H*V], beta [T, H] (before its sigmoid): views of one dtype with free row
+    strides; z fp32 [T, H*D]; dt_bias fp32 [H*D], a_log fp32 [H]; state fp32 [slots, H, V, D]."""
+    _gpu(o, q, k, v, beta, z, dt_bias, a_log, state, query_start_loc, context_lens, state_slots)
+    slots, H, V, D = state.shape
+    T, B = q.shape[0], context_lens.numel()
+    assert o.dtype == torch.float32 and o.is_contiguous() and o.shape == (T, H * V)
+    assert state.dtype == torch.float32 and state.is_contiguous() and z.dtype == torch.float32
+    assert q.dtype == k.dtype == v.dtype == beta.dtype
+    for t in (dt_bias, a_log):
+        assert t.dtype == torch.float32 and t.is_contiguous()
+    assert dt_bias.numel() == H * D and a_log.numel() == H
+    for t in (query_start_loc, context_lens, state_slots):
+        assert t.dtype == torch.int32 and t.is_contiguous()
+    assert query_start_loc.numel() == B + 1 and state_slots.numel() == B
+    L = _lib.seq_lib()
+    need = L.vla_seq_channel_delta_scratch_floats(T, B, int(max_query_len), H, D, V)
+    scratch = torch.empty(need, dtype=torch.float32, device=q.device) if need else None
+    with torch.cuda.device(q.device):
+        seq_check(L.vla_seq_channel_delta_scan(
+            o.data_ptr(), q.data_ptr(), _rows(q, kv_heads * D), k.data_ptr(), _rows(k, kv_heads * D), v.data_ptr(),
+            _rows(v, H * V), beta.data_ptr(), _rows(beta, H), z.data_ptr(), _rows(z, H * D), dt_bias.data_ptr(),
+            a_log.data_ptr(), state.data_ptr(), query_start_loc.data_ptr(), context_lens.data_ptr(),
+            state_slots.data_ptr(), T, B, slots, int(max_query_len), H, int(kv_heads), D, V, _p(scratch), need,
+            _dt(q.dtype), _stream(q.device)), "channel_delta_scan")
+
+
+def set_channel_delta_kernel(mode: int) -> None:
+    """0: channel_delta_scan picks its kernel per run of rows; 1: always token by token; 2: always in blocks."""
+    seq_check(_lib.seq_lib().vla_seq_set_channel_delta_kernel(mode), "set_channel_delta_kernel")
+
+
 # ---------------------------------------------------------------- recurrences with one decay per head
 def decay_scan(o: torch.Tensor, q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, state: torch.Tensor,
                query_start_loc: torch.Tensor, context_lens: torch.Tensor, state_slots: torch.Tensor, groups: int,
                max_query_len: int, log_decay: Optional[torch.Tensor] = None, dt: Optional[torch.Tensor] = None,
                dt_bias: Optional[torch.Tensor] = None, a_log: Optional[torch.Tensor] = None,
-               skip: Optional[torch.Tensor] = None, act: str = "none") -> None:
+               skip: Optional[torch.Tensor] = None, act: str = "none", row_log: Optional[torch.Tensor] = None,
+               row_weight: Optional[torch.Tensor] = None, row_floor: Optional[torch.Tensor] = None,
+               norm_scale: Optional[torch.Tensor] = None, norm_eps: float = 0.0, q_scale: float = 1.0,
+               sizes: Optional[tuple] = None) -> None:
     """Per head S <- e^g S + w k v^T, o = S^T q + skip v; g = log_decay[h] and w = 1, or w = softplus(dt +
-    dt_bias) and g = -exp(a_log) w; q, k, v pass `act` ("none" or "silu") first.  o fp32 [T, H*V];
-    q, k [T, groups*D], v [T, H*V], dt [T, H]: views with free row strides; log_decay, dt_bias, a_log,
-    skip fp32 [H]; state fp32 [slots, H, D, V]."""
-    _gpu(o, q, k, v, state, query_start_loc, context_lens, state_slots, log_decay, dt, dt_bias, a_log, skip)
-    slots, H, D, V = state.shape
+    dt_bias) and g = -exp(a_log) w, or g = row_log[t, h] and w = row_weight[t, h]; q, k, v pass `act` ("none"
+    or "silu") first, q then times q_scale.  o fp32 [T, H*V]; q, k [T, groups*D], v [T, H*V], dt [T, H]:
+    views with free row strides; log_decay, dt_bias, a_log, skip fp32 [H]; state fp32 [slots, H, D, V].
+    norm_scale (fp32 [T, H], written): a normalizer n <- e^g n + w k runs along and norm_scale =
+    1 / (max(|n . q|, row_floor[t, h]) + norm_eps); then sizes = (D, V) and the state is fp32
+    [slots, H, D * (V + 1)], a head's S followed by its n."""
+    _gpu(o, q, k, v, state, query_start_loc, context_lens, state_slots, log_decay, dt, dt_bias, a_log, skip, row_log,
+         row_weight, row_floor, norm_scale)
+    if norm_scale is None:
+        slots, H, D, V = state.shape
+    else:
+        (slots, H, size), (D, V) = state.shape, sizes
+        assert size == D * (V + 1) and row_floor is not None
     T, B = q.shape[0], context_lens.numel()
     assert o.dtype == torch.float32 and o.is_contiguous() and o.shape == (T, H * V)
     assert state.dtype == torch.float32 and state.is_contiguous()
     assert q.dtype == k.dtype == v.dtype and (dt is None or dt.dtype == q.dtype)
-    assert (dt is None) != (log_decay is None) and (dt is None or (dt_bias is not None and a_log is not None))
+    assert sum(t is not None for t in (dt, log_decay, row_log)) == 1 and (row_log is None) == (row_weight is None)
+    assert dt is None or (dt_bias is not None and a_log is not None)
+    for t in (row_log, row_weight, row_floor, norm_scale):
+        assert t is None or (t.dtype == torch.float32 and t.shape == (T, H) and t.is_contiguous())
     for t in (log_decay, dt_bias, a_log, skip):
         assert t is None or (t.dtype == torch.float32 and t.numel() == H and t.is_contiguous())
     for t in (query_start_loc, context_lens, state_slots):
         assert t.dtype == torch.int32 and t.is_contiguous()
     assert query_start_loc.numel() == B + 1 and state_slots.numel() == B
     L = _lib.seq_lib()
-    need = L.vla_seq_decay_scan_scratch_floats(T, B, int(max_query_len), H, D, V)
+    need = L.vla_seq_decay_scan_scratch_floats(T, B, int(max_query_len), H, D, V, int(norm_scale is not None))
     scratch = torch.empty(need, dtype=torch.float32, device=q.device) if need else None
     with torch.cuda.device(q.device):
         seq_check(L.vla_seq_decay_scan(
             o.data_ptr(), q.data_ptr(), _rows(q, groups * D), k.data_ptr(), _rows(k, groups * D), v.data_ptr(),
             _rows(v, H * V), _p(dt), 0 if dt is None else _rows(dt, H), _p(dt_bias), _p(a_log), _p(log_decay),
-            _p(skip), state.data_ptr(), query_start_loc.data_ptr(), context_lens.data_ptr(), state_slots.data_ptr(),
+            _p(skip), _p(row_log), _p(row_weight), _p(row_floor), _p(norm_scale), float(norm_eps), float(q_scale),
+            state.data_ptr(), query_start_loc.data_ptr(), context_lens.data_ptr(), state_slots.data_ptr(),
             T, B, slots, int(max_query_len), H, int(groups), D, V, ACT[act], _p(scratch), need, _dt(q.dtype),
             _stream(q.device)), "decay_scan")
 
@@ -777,19 +860,47 @@ def set_decay_scan_kernel(mode: int) -> None:
 
 
 def gated_group_rms_norm(out: torch.Tensor, o: torch.Tensor, weight: torch.Tensor, gate: torch.Tensor, gate_act: str,
-                         gate_first: bool, groups: int, eps: float) -> None:
+                         gate_first: bool, groups: int, eps: float, part_scale: Optional[torch.Tensor] = None) -> None:
     """gate_first: u = o * gate_act(gate), out = u / rms(u) * weight; else out = o / rms(o) * weight *
     gate_act(gate); the norm runs over each of `groups` equal parts of a row.  o fp32 [T, n]; gate, out
-    [T, n] views with free row strides; gate_act "silu" or "sigmoid"."""
-    _gpu(out, o, weight, gate)
+    [T, n] views with free row strides; gate_act "silu" or "sigmoid"; part_scale fp32 [T, groups]
+    multiplies every part of o first."""
+    _gpu(out, o, weight, gate, part_scale)
+    assert part_scale is None or (part_scale.dtype == torch.float32 and part_scale.is_contiguous() and
+                                  part_scale.shape == (o.shape[0], groups))
     T, n = o.shape
     assert o.dtype == torch.float32 and o.is_contiguous() and out.dtype == gate.dtype
     assert weight.dtype == torch.float32 and weight.numel() == n and weight.is_contiguous()
     with torch.cuda.device(o.device):
         seq_check(_lib.seq_lib().vla_seq_gated_group_rms_norm(
             out.data_ptr(), _rows(out, n), o.data_ptr(), weight.data_ptr(), gate.data_ptr(), _rows(gate, n),
-            GATE[gate_act], int(bool(gate_first)), int(groups), float(eps), T, n, _dt(out.dtype), _stream(o.device)),
-            "gated_group_rms_norm")
+            GATE[gate_act], int(bool(gate_first)), int(groups), float(eps), T, n, _dt(out.dtype), _p(part_scale),
+            _stream(o.device)), "gated_group_rms_norm")
+
+
+def matrix_memory_gates(zi: torch.Tensor, zf: torch.Tensor, bias_i: torch.Tensor, bias_f: torch.Tensor, cap: float,
+                        maximum: torch.Tensor, query_start_loc: torch.Tensor, context_lens: torch.Tensor,
+                        state_slots: torch.Tensor, max_query_len: int):
+    """Capped exponential gates with a running maximum m (fp32 [slots, H], brought up to date): i = cap
+    tanh((zi + bias_i) / cap), f = log sigmoid(cap tanh((zf + bias_f) / cap)), m_t = max(f + m_(t-1), i).  zi,
+    zf [T, H] views.  -> fp32 [T, H] each: f + m_(t-1) - m_t, e^(i - m_t), e^(-m_t)."""
+    _gpu(zi, zf, bias_i, bias_f, maximum, query_start_loc, context_lens, state_slots)
+    T, H = zi.shape
+    slots, B = maximum.shape[0], context_lens.numel()
+    assert zf.shape == (T, H) and zf.dtype == zi.dtype and maximum.shape == (slots, H)
+    for t in (bias_i, bias_f, maximum):
+        assert t.dtype == torch.float32 and t.is_contiguous() and t.shape[-1] == H
+    for t in (query_start_loc, context_lens, state_slots):
+        assert t.dtype == torch.int32 and t.is_contiguous()
+    assert query_start_loc.numel() == B + 1 and state_slots.numel() == B
+    out = torch.empty((3, T, H), dtype=torch.float32, device=zi.device)
+    with torch.cuda.device(zi.device):
+        seq_check(_lib.seq_lib().vla_seq_matrix_memory_gates(
+            out[0].data_ptr(), out[1].data_ptr(), out[2].data_ptr(), zi.data_ptr(), _rows(zi, H), zf.data_ptr(),
+            _rows(zf, H), bias_i.data_ptr(), bias_f.data_ptr(), float(cap), maximum.data_ptr(),
+            query_start_loc.data_ptr(), context_lens.data_ptr(), state_slots.data_ptr(), B, slots, int(max_query_len), H,
+            _dt(zi.dtype), _stream(zi.device)), "matrix_memory_gates")
+    return out[0], out[1], out[2]
 
 
 def rglru_scan(out: torch.Tensor, gates: torch.Tensor, u: torch.Tensor, y: torch.Tensor,
@@ -849,11 +960,14 @@ def latent_rotary_write(q: torch.Tensor, q_head_stride: int, q_first: int, heads
 
 def latent_attention(out: torch.Tensor, q_lat: torch.Tensor, q_rot: torch.Tensor, cache: torch.Tensor,
                      block_tables: torch.Tensor, token_seq: torch.Tensor, positions: torch.Tensor,
-                     scale: float, window: int = 0, gate: Optional[torch.Tensor] = None) -> None:
+                     scale: float, window: int = 0, gate: Optional[torch.Tensor] = None,
+                     sinks: Optional[torch.Tensor] = None) -> None:
     """out, q_lat [T, H, rank] and q_rot [T, H, rot] views (any token / head strides, unit stride
     along the last axis); cache [NB, BS, rank + rot]; window > 0: keys with position - j < window
-    only; gate [T, H]: a head's sums times sigmoid(gate)."""
-    _gpu(out, q_lat, q_rot, cache, block_tables, token_seq, positions, gate)
+    only; gate [T, H]: a head's sums times sigmoid(gate); sinks fp32 [H]: e^sink joins a head's
+    softmax denominator."""
+    _gpu(out, q_lat, q_rot, cache, block_tables, token_seq, positions, gate, sinks)
+    assert sinks is None or (sinks.dtype == torch.float32 and sinks.numel() == q_lat.shape[1] and sinks.is_contiguous())
     assert gate is None or gate.dtype == q_lat.dtype
     NB, BS, width = cache.shape
     T, H, rank = q_lat.shape
@@ -870,7 +984,7 @@ def latent_attention(out: torch.Tensor, q_lat: torch.Tensor, q_rot: torch.Tensor
             out.data_ptr(), out.stride(0), out.stride(1), q_lat.data_ptr(), q_lat.stride(0), q_lat.stride(1),
             q_rot.data_ptr(), q_rot.stride(0), q_rot.stride(1), cache.data_ptr(), block_tables.data_ptr(),
             block_tables.shape[1], token_seq.data_ptr(), positions.data_ptr(), T, H, rank, rot, BS, NB, float(scale),
-            _dt(q_lat.dtype), int(window), _p(gate), 0 if gate is None else _rows(gate, H),
+            _dt(q_lat.dtype), int(window), _p(gate), 0 if gate is None else _rows(gate, H), _p(sinks),
             _stream(q_lat.device)), "latent_attention")
 
 
@@ -893,11 +1007,12 @@ def latent_attention_tiles_supported(q_lat: torch.Tensor, q_rot: torch.Tensor, c
 def latent_attention_tiles(out: torch.Tensor, q_lat: torch.Tensor, q_rot: torch.Tensor, cache: torch.Tensor,
                            block_tables: torch.Tensor, query_start_loc: torch.Tensor, context_lens: torch.Tensor,
                            max_query_len: int, scale: float, key_splits: int = 1, window: int = 0,
-                           gate: Optional[torch.Tensor] = None) -> None:
+                           gate: Optional[torch.Tensor] = None, sinks: Optional[torch.Tensor] = None) -> None:
     """The same attention as latent_attention for 16-bit activations on the matrix cores; rows
     query_start_loc[b] .. of sequence b sit at positions context_lens[b] ...  key_splits > 1: the
     keys of every row tile are shared out to that many workgroups and merged."""
-    _gpu(out, q_lat, q_rot, cache, block_tables, query_start_loc, context_lens, gate)
+    _gpu(out, q_lat, q_rot, cache, block_tables, query_start_loc, context_lens, gate, sinks)
+    assert sinks is None or (sinks.dtype == torch.float32 and sinks.numel() == q_lat.shape[1] and sinks.is_contiguous())
     NB, BS, width = cache.shape
     T, H, rank = q_lat.shape
     rot = width - rank
@@ -923,5 +1038,5 @@ def latent_attention_tiles(out: torch.Tensor, q_lat: torch.Tensor, q_rot: torch.
             q_rot.data_ptr(), st(q_rot, 0), st(q_rot, 1), cache.data_ptr(), block_tables.data_ptr(),
             block_tables.shape[1], query_start_loc.data_ptr(), context_lens.data_ptr(), B, int(max_query_len), H, rank,
             rot, BS, NB, float(scale), int(key_splits), _p(scratch), T, _dt(q_lat.dtype), int(window), _p(gate),
-            0 if gate is None else _rows(gate, H), _stream(q_lat.device)),
+            0 if gate is None else _rows(gate, H), _p(sinks), _stream(q_lat.device)),
             "latent_attention_tiles")

@@ -309,3 +309,87 @@ class StateSpaceRecurrence(nn.Module):
                        dt_bias=self.dt_bias.data, a_log=self.a_log.data, skip=self.skip.data)
         ops.gated_group_rms_norm(out, y, self.norm_weight.data, z, "silu", True, self.norm_groups, self.eps)
         return out
+
+
+class ChannelDeltaRule(nn.Module):
+    """Delta rule with a decay per key channel and per-sequence state slots.  Per head, on a state S
+    [dim, vdim]:  S <- diag(g) S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q, with k and q unit
+    vectors per key head (q also times dim^-1/2; `heads / kv_heads` value heads share one), beta =
+    sigmoid(b) and g = exp(-exp(A_log) softplus(z + dt_bias)) per head and channel; o leaves RMS-normed over
+    vdim, weighted (one weight vector for all heads) and times sigmoid(gate).  The state is fp32
+    [num_slots, heads, vdim, dim] and a sequence whose context length is 0 starts from zero whatever its
+    slot held (csrc/seq_channel_delta.hip)."""
+
+    def __init__(self, heads: int, kv_heads: int, dim: int, vdim: int, eps: float, device=None) -> None:
+        super().__init__()
+        if heads % kv_heads:
+            raise ValueError("heads is not a multiple of kv_heads")
+        self.heads, self.kv_heads, self.dim, self.vdim, self.eps = heads, kv_heads, dim, vdim, float(eps)
+
+        def par(n, fill=0.0):
+            return nn.Parameter(torch.full((n, ), fill, dtype=torch.float32, device=device), requires_grad=False)
+
+        self.a_log, self.dt_bias, self.norm_weight = par(heads), par(heads * dim), par(heads * vdim, 1.0)
+
+    def set_weights(self, a_log: torch.Tensor, dt_bias: torch.Tensor, norm_weight: torch.Tensor) -> None:
+        """a_log [heads], dt_bias [heads * dim], norm_weight [vdim] (repeated for every head)."""
+        dev = self.a_log.device
+        self.a_log.data, self.dt_bias.data = a_log.float().to(dev).contiguous(), dt_bias.float().to(dev).contiguous()
+        self.norm_weight.data = norm_weight.float().repeat(self.heads).to(dev).contiguous()
+
+    @staticmethod
+    def get_state_shape(num_slots: int, heads: int, dim: int, vdim: int) -> Tuple[int, ...]:
+        return (num_slots, heads, vdim, dim)
+
+    def forward(self, out: torch.Tensor, q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, gate: torch.Tensor,
+                beta: torch.Tensor, z: torch.Tensor, state: torch.Tensor, batch: SequenceBatch) -> torch.Tensor:
+        """q, k [T, G*D], v, gate, out [T, H*V], beta [T, H], z fp32 [T, H*D]: views with free row strides."""
+        o = torch.empty((q.shape[0], self.heads * self.vdim), dtype=torch.float32, device=q.device)
+        ops.channel_delta_scan(o, q, k, v, beta, z, self.dt_bias.data, self.a_log.data, state, batch.query_start_loc,
+                               batch.context_lens, batch.state_slots, self.kv_heads, batch.max_query_len)
+        ops.gated_group_rms_norm(out, o, self.norm_weight.data, gate, "sigmoid", False, self.heads, self.eps)
+        return out
+
+
+class MatrixMemory(nn.Module):
+    """Matrix memory with exponential gates (the mLSTM of xLSTM) and per-sequence state slots.  Per head
+    S_t = e^f S_(t-1) + e^i k v^T and n_t = e^f n_(t-1) + e^i k, both kept times e^(-m_t) with the running
+    maximum m_t = max(f + m_(t-1), i) from 0 on; o = S^T q / (max(|n . q|, e^(-m)) + 1e-6) with q times
+    dim^-1/2.  The log gates are i = cap tanh((zi + bias_i) / cap) and f = log sigmoid(cap tanh((zf + bias_f)
+    / cap)).  Each head's o is divided by its root mean square, weighted per element and times
+    sigmoid(gate).  State: fp32 [num_slots, heads, dim * (vdim + 1)] (S, then n) and the maximum fp32
+    [num_slots, heads]; a sequence whose context length is 0 starts from zero (csrc/seq_decay_scan.hip)."""
+
+    NORM_EPS = 1e-6
+
+    def __init__(self, heads: int, dim: int, vdim: int, gate_cap: float, eps: float, device=None) -> None:
+        super().__init__()
+        if not gate_cap > 0:
+            raise ValueError("the gates' cap must be positive")
+        self.heads, self.dim, self.vdim, self.gate_cap, self.eps = heads, dim, vdim, float(gate_cap), float(eps)
+
+        def par(n, fill=0.0):
+            return nn.Parameter(torch.full((n, ), fill, dtype=torch.float32, device=device), requires_grad=False)
+
+        self.bias_i, self.bias_f, self.norm_weight = par(heads), par(heads), par(heads * vdim, 1.0)
+
+    @staticmethod
+    def get_state_shapes(num_slots: int, heads: int, dim: int, vdim: int) -> Tuple[Tuple[int, ...], Tuple[int, ...]]:
+        """(memory and normalizer, running maximum)."""
+        return (num_slots, heads, dim * (vdim + 1)), (num_slots, heads)
+
+    def forward(self, out: torch.Tensor, q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, gate: torch.Tensor,
+                zi: torch.Tensor, zf: torch.Tensor, memory: torch.Tensor, maximum: torch.Tensor,
+                batch: SequenceBatch) -> torch.Tensor:
+        """q, k [T, H*D], v, gate, out [T, H*V], zi, zf [T, H] (one dtype): views with free row strides."""
+        T, H = q.shape[0], self.heads
+        row_log, row_weight, row_floor = ops.matrix_memory_gates(
+            zi, zf, self.bias_i.data, self.bias_f.data, self.gate_cap, maximum, batch.query_start_loc,
+            batch.context_lens, batch.state_slots, batch.max_query_len)
+        o = torch.empty((T, H * self.vdim), dtype=torch.float32, device=q.device)
+        norm_scale = torch.empty((T, H), dtype=torch.float32, device=q.device)
+        ops.decay_scan(o, q, k, v, memory, batch.query_start_loc, batch.context_lens, batch.state_slots, H,
+                       batch.max_query_len, row_log=row_log, row_weight=row_weight, row_floor=row_floor,
+                       norm_scale=norm_scale, norm_eps=self.NORM_EPS, q_scale=self.dim**-0.5, sizes=(self.dim, self.vdim))
+        ops.gated_group_rms_norm(out, o, self.norm_weight.data, gate, "sigmoid", False, H, self.eps, norm_scale)
+        return out

@@ -1,8 +1,20 @@
 // Linear recurrence with one decay per head and token, on an fp32 state S [dim, vdim] per head:
 //   S <- e^g S + w k v^T;   o = S^T q + skip v
 // g and w come from a step size (w = softplus(dt + dt_bias), g = -exp(a_log) w: a state-space layer whose
-// heads share queries and keys by group) or are constant (g = log_decay[head], w = 1).  q, k and v may
-// pass an activation on their way in.
+// heads share queries and keys by group), are constant (g = log_decay[head], w = 1) or are given per row
+// (a matrix memory with exponential gates: matrix_memory_gates forms them).  q, k and v may pass an
+// activation on their way in; q may be scaled.
+//
+// Normalizer (a matrix memory): beside S a vector n [dim] runs through the same recurrence with the value
+// 1 -- its product with the query is the row sum of P plus the part of the block's start, so it costs no
+// product -- and the scan leaves 1 / (max(|n . q|, floor) + eps) per (token, head) for whoever reads o.
+// A head's state is then S followed by n.
+//
+// matrix_memory_gates: log input gate i = cap tanh((zi + bi) / cap), log forget gate
+// f = -softplus(-cap tanh((zf + bf) / cap)), running maximum m_t = max(f + m_(t-1), i) from 0 on; what
+// the scan needs is g = f + m_(t-1) - m_t <= 0, w = e^(i - m_t) <= 1 and the floor e^(-m_t).  S and n are
+// scaled by e^(-m_t), so any rounding of m cancels as long as g, w and the floor come from the same
+// numbers.  m -> max(a + m, b) composes, so a workgroup scans its rows in log steps.
 //
 // Blocks of 64 rows (runs of more than a few rows).  With c_i the sum of g over a block's rows 0 .. i,
 //   o_i = e^(c_i) S^T q_i + sum_(j <= i) e^(c_i - c_j) w_j (q_i . k_j) v_j + skip v_i
@@ -66,8 +78,14 @@ struct DecayScan {
   const float* a_log;
   const float* log_decay;
   const float* skip;
+  const float* row_log;       // [T][heads]: g per row
+  const float* row_weight;    // [T][heads]: w per row
+  const float* row_floor;     // [T][heads]
+  float* norm_scale;          // [T][heads]; null: no normalizer
+  float norm_eps, q_scale;
+  int64_t head_size;          // state numbers per head: dim * vdim, plus dim with a normalizer
   float* state;
-  float* piece_state;     // [piece slots][heads][dim][vdim]
+  float* piece_state;     // [piece slots][heads][head_size]
   float* piece_decay;     // [piece slots][heads]
   const int* query_start_loc;
   const int* context_lens;
@@ -83,10 +101,28 @@ __device__ __forceinline__ float load_one(const void* p, int64_t i, int dtype) {
   return ((const float*)p)[i];
 }
 
-// the log decay and the input's factor of a row (dt: its step size's projection, where there is one)
-__device__ __forceinline__ void row_decay(const DecayScan& a, float dt, int h, float& g, float& w) {
-  if (a.dt != nullptr) {
-    w = softplus_f(dt + a.dt_bias[h]);
+// what a row's decay comes from: its step size's projection, or its log decay and weight
+struct RowDecay {
+  float dt = 0.f, weight = 0.f;
+};
+__device__ __forceinline__ RowDecay load_decay(const DecayScan& a, int64_t t, int h) {
+  RowDecay r;
+  if (a.row_log != nullptr) {
+    r.dt = a.row_log[t * a.heads + h];
+    r.weight = a.row_weight[t * a.heads + h];
+  } else if (a.dt != nullptr) {
+    r.dt = load_one(a.dt, t * a.dt_stride + h, a.dtype);
+  }
+  return r;
+}
+
+// the log decay and the input's factor of a row
+__device__ __forceinline__ void row_decay(const DecayScan& a, const RowDecay& r, int h, float& g, float& w) {
+  if (a.row_log != nullptr) {
+    w = r.weight;
+    g = fminf(r.dt, 0.f);
+  } else if (a.dt != nullptr) {
+    w = softplus_f(r.dt + a.dt_bias[h]);
     g = -expf(a.a_log[h]) * w;
   } else {
     w = 1.f;
@@ -225,7 +261,8 @@ enum RowKind {
 template <int DB, int WAVES, RowKind KIND, bool STATE_ONLY>
 constexpr size_t block_lds_floats() {
   constexpr int DP = 16 * DB, QK = KIND == kRowsBf16 ? (DP + 8) / 2 : DP + 4;     // floats per query / key row
-  return (size_t)kBlock * ((STATE_ONLY ? 1 : 2) * QK + (16 * WAVES + 4) + (STATE_ONLY ? 0 : kBlock + 4)) + 5 * kBlock;
+  return (size_t)kBlock * ((STATE_ONLY ? 1 : 2) * QK + (16 * WAVES + 4) + (STATE_ONLY ? 0 : kBlock + 4)) + 5 * kBlock +
+         2 * DP;
 }
 
 template <int DB, int WAVES, RowKind KIND, bool STATE_ONLY>
@@ -242,8 +279,9 @@ __global__ __launch_bounds__(64 * WAVES) void decay_block_kernel(DecayScan a) {
   E* k_lds = reinterpret_cast<E*>(lds);                 // [64][KR]
   float* v_lds = lds + kBlock * QK_FLOATS;              // [64][VR]
   float* num = v_lds + kBlock * VR;                     // c | w | e^c | e^(c_last - c) w | c's low part
-  E* q_lds = reinterpret_cast<E*>(num + 5 * kBlock);    // [64][KR]
-  float* p_lds = num + 5 * kBlock + kBlock * QK_FLOATS; // [64][PR]
+  float* n_lds = num + 5 * kBlock;                      // [2][DP] the normalizer, before / after a block
+  E* q_lds = reinterpret_cast<E*>(n_lds + 2 * DP);      // [64][KR]
+  float* p_lds = n_lds + 2 * DP + kBlock * QK_FLOATS;   // [64][PR]
   const int h = blockIdx.x, v0 = blockIdx.y * VB, z = blockIdx.z;
   int b, piece;
   if (!find_piece(a, z, b, piece)) return;
@@ -257,7 +295,8 @@ __global__ __launch_bounds__(64 * WAVES) void decay_block_kernel(DecayScan a) {
   const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6, g = lane >> 4, c = lane & 15;
   const int D = a.dim, V = a.vdim, hg = h / (a.heads / a.groups);
   const int v_mine = v0 + 16 * w + c;                   // this lane's value column
-  const int64_t state_size = (int64_t)D * V;
+  const int64_t state_size = a.head_size;
+  const bool normed = a.norm_scale != nullptr && blockIdx.y == 0;   // one workgroup of a head keeps n
   const float* from = nullptr;
   if (!STATE_ONLY) {
     if (cut)
@@ -273,11 +312,14 @@ __global__ __launch_bounds__(64 * WAVES) void decay_block_kernel(DecayScan a) {
       const int d = 16 * db + 4 * g + r;
       s[db][r] = from != nullptr && d < D && v_mine < V ? from[(int64_t)d * V + v_mine] : 0.f;
     }
-  const float skip = a.skip != nullptr && !STATE_ONLY ? a.skip[h] : 0.f;
+  if (normed)
+    for (int d = tid; d < DP; d += THREADS) n_lds[d] = from != nullptr && d < D ? from[(int64_t)D * V + d] : 0.f;
+  int n_at = 0;
+  const float skip = a.skip != nullptr && !STATE_ONLY ? a.skip[h] : 0.f, q_scale = a.q_scale;
   double log_total = 0.0;
 
   Piece<W16> pq[NQ], pk[NQ], pv[NVP];
-  float row_dt = 0.f;
+  RowDecay row_next;
   auto fetch = [&](int t0) {
     const int n = min(kBlock, t_end - t0);
 #pragma unroll
@@ -292,8 +334,7 @@ __global__ __launch_bounds__(64 * WAVES) void decay_block_kernel(DecayScan a) {
       const int i = tid + THREADS * u, r = i / (VB / 8), d = v0 + 8 * (i % (VB / 8));
       pv[u] = read_piece<W16>(a.v, (int64_t)(t0 + min(r, n - 1)) * a.v_stride + (int64_t)h * V, d, V, a.vec_v);
     }
-    if (tid < kBlock && a.dt != nullptr)
-      row_dt = load_one(a.dt, (int64_t)(t0 + min(tid, n - 1)) * a.dt_stride + h, a.dtype);
+    if (tid < kBlock) row_next = load_decay(a, t0 + min(tid, n - 1), h);
   };
   auto land_qk = [&](E* dst, Piece<W16>& p, bool live) {
     mask_piece<W16>(p, live);
@@ -305,7 +346,7 @@ __global__ __launch_bounds__(64 * WAVES) void decay_block_kernel(DecayScan a) {
   auto land = [&](int n) {
     if (w == 0) {
       float row_g = 0.f, row_w = 0.f;
-      if (lane < n) row_decay(a, row_dt, h, row_g, row_w);
+      if (lane < n) row_decay(a, row_next, h, row_g, row_w);
       double cs = row_g;                                // inclusive sum over the 64 rows
 #pragma unroll
       for (int m = 1; m < 64; m <<= 1) {
@@ -385,10 +426,29 @@ __global__ __launch_bounds__(64 * WAVES) void decay_block_kernel(DecayScan a) {
         for (int r = 0; r < 4; ++r) {
           const int i = 16 * ib + 4 * g + r;
           const float diff = fminf((num[i] - cj) + (num[4 * kBlock + i] - lj), 0.f);
-          p_lds[i * PR + j] = j <= i ? acc[r] * (expf(diff) * wj) : 0.f;
+          p_lds[i * PR + j] = j <= i ? acc[r] * (expf(diff) * wj * q_scale) : 0.f;
         }
       }
       __syncthreads();
+      if (normed) {
+        // n . q of every row: PARTS neighbouring threads share one
+        constexpr int PARTS = THREADS / kBlock;
+        const int i = tid / PARTS, part = tid % PARTS;
+        float dot = 0.f, sum = 0.f;
+        for (int d = 4 * part; d < DP; d += 4 * PARTS) {
+          const f32x4 qv = four(q_lds + i * KR + d), nv = *reinterpret_cast<const f32x4*>(n_lds + n_at * DP + d);
+#pragma unroll
+          for (int e = 0; e < 4; ++e) dot += qv[e] * nv[e];
+        }
+        for (int j = part; j <= i; j += PARTS) sum += p_lds[i * PR + j];
+        sum += dot * (num[2 * kBlock + i] * q_scale);
+#pragma unroll
+        for (int m = 1; m < PARTS; m <<= 1) sum += __shfl_xor(sum, m, 64);
+        if (part == 0 && i < n) {
+          const int64_t at = (int64_t)(t0 + i) * a.heads + h;
+          a.norm_scale[at] = 1.f / (fmaxf(fabsf(sum), a.row_floor[at]) + a.norm_eps);
+        }
+      }
     }
     // this wave's value columns as B operands: rows 16 kb + 4 g + i
     float vf[4][4];
@@ -409,7 +469,7 @@ __global__ __launch_bounds__(64 * WAVES) void decay_block_kernel(DecayScan a) {
           }
           const f32x4 ec = *reinterpret_cast<const f32x4*>(num + 2 * kBlock + 16 * rb + 4 * g);
 #pragma unroll
-          for (int r = 0; r < 4; ++r) acc[r] = acc[r] * ec[r] + skip * vf[rb][r];
+          for (int r = 0; r < 4; ++r) acc[r] = acc[r] * (ec[r] * q_scale) + skip * vf[rb][r];
 #pragma unroll
           for (int kb = 0; kb <= rb; ++kb) {
             const f32x4 pa = *reinterpret_cast<const f32x4*>(p_lds + (16 * rb + c) * PR + 16 * kb + 4 * g);
@@ -425,6 +485,15 @@ __global__ __launch_bounds__(64 * WAVES) void decay_block_kernel(DecayScan a) {
       }
     }
     const float e_last = num[2 * kBlock + kBlock - 1];
+    if (normed) {                                        // readers of the other half are behind the last barrier
+      for (int d = tid; d < DP; d += THREADS) {
+        float nv = e_last * n_lds[n_at * DP + d];
+#pragma unroll 8
+        for (int j = 0; j < kBlock; ++j) nv += num[3 * kBlock + j] * one(k_lds + j * KR + d);
+        n_lds[(1 - n_at) * DP + d] = nv;
+      }
+      n_at = 1 - n_at;
+    }
     log_total += (double)num[kBlock - 1] + (double)num[5 * kBlock - 1];
 #pragma unroll
     for (int kb = 0; kb < 4; ++kb) {
@@ -462,6 +531,8 @@ __global__ __launch_bounds__(64 * WAVES) void decay_block_kernel(DecayScan a) {
       const int d = 16 * db + 4 * g + r;
       if (d < D && v_mine < V) to[(int64_t)d * V + v_mine] = s[db][r];
     }
+  if (normed)                                            // written before the last barrier
+    for (int d = tid; d < D; d += THREADS) to[(int64_t)D * V + d] = n_lds[n_at * DP + d];
 }
 
 // Over one sequence's pieces: what piece i leaves from zero (in its slot) becomes what it starts from.
@@ -472,7 +543,7 @@ __global__ __launch_bounds__(256) void decay_chain_kernel(DecayScan a) {
   if (run <= a.piece_rows) return;
   const int count = (run + a.piece_rows - 1) / a.piece_rows;
   const int z0 = a.query_start_loc[b] / a.piece_rows + b;
-  const int64_t size = (int64_t)a.dim * a.vdim;
+  const int64_t size = a.head_size;
   const int64_t e = (int64_t)blockIdx.x * 256 + threadIdx.x;
   if (e >= size) return;
   float s = a.context_lens[b] > 0 ? a.state[((int64_t)a.state_slots[b] * a.heads + h) * size + e] : 0.f;
@@ -512,7 +583,10 @@ __global__ __launch_bounds__(256) void decay_step_kernel(DecayScan a) {
   float* k_lds = q_lds + D;              // [D]
   float* v_lds = k_lds + D;              // [V]
   float* part = v_lds + V;               // [groups][V]
-  float* st = a.state + ((int64_t)a.state_slots[b] * a.heads + h) * (int64_t)D * V + VW * cg;
+  float* red = part + groups * V;        // [4]
+  float* head = a.state + ((int64_t)a.state_slots[b] * a.heads + h) * a.head_size;
+  float* st = head + VW * cg;
+  float* n_st = head + (int64_t)D * V;
   const bool resume = a.context_lens[b] > 0;
   const float skip = a.skip != nullptr ? a.skip[h] : 0.f;
   auto load = [&](const void* p, int64_t i) {
@@ -521,15 +595,25 @@ __global__ __launch_bounds__(256) void decay_step_kernel(DecayScan a) {
   };
   for (int t = t_begin; t < t_end; ++t) {
     float g, wt;
-    row_decay(a, a.dt != nullptr ? load_one(a.dt, (int64_t)t * a.dt_stride + h, a.dtype) : 0.f, h, g, wt);
+    row_decay(a, load_decay(a, t, h), h, g, wt);
     const float e = expf(g);
     for (int d = tid; d < D; d += 256) {
-      q_lds[d] = load(a.q, (int64_t)t * a.q_stride + (int64_t)hg * D + d);
+      q_lds[d] = load(a.q, (int64_t)t * a.q_stride + (int64_t)hg * D + d) * a.q_scale;
       k_lds[d] = load(a.k, (int64_t)t * a.k_stride + (int64_t)hg * D + d);
     }
     for (int d = tid; d < V; d += 256) v_lds[d] = load(a.v, (int64_t)t * a.v_stride + (int64_t)h * V + d);
     __syncthreads();
     const bool zero = !resume && t == t_begin;
+    if (a.norm_scale != nullptr) {
+      float dot = 0.f;
+      for (int d = tid; d < D; d += 256) {
+        const float nv = (zero ? 0.f : e * n_st[d]) + wt * k_lds[d];
+        n_st[d] = nv;
+        dot += q_lds[d] * nv;
+      }
+      dot = wave_sum(dot);
+      if ((tid & 63) == 0) red[tid >> 6] = dot;
+    }
     float o[VW], wv[VW];
 #pragma unroll
     for (int x = 0; x < VW; ++x) {
@@ -578,8 +662,122 @@ __global__ __launch_bounds__(256) void decay_step_kernel(DecayScan a) {
       for (int r = 0; r < groups; ++r) sum += part[r * V + v];
       a.o[((int64_t)t * a.heads + h) * V + v] = sum;
     }
+    if (a.norm_scale != nullptr && tid == 0) {
+      const int64_t at = (int64_t)t * a.heads + h;
+      a.norm_scale[at] = 1.f / (fmaxf(fabsf(red[0] + red[1] + red[2] + red[3]), a.row_floor[at]) + a.norm_eps);
+    }
     __syncthreads();
   }
+}
+
+__device__ __forceinline__ float capped(float z, float cap) { return cap * tanhf(z / cap); }
+
+// One workgroup per (head, sequence): each thread one row of a stretch of blockDim.x.
+template <class S>
+__global__ __launch_bounds__(1024) void matrix_memory_gates_kernel(
+    float* __restrict__ row_log, float* __restrict__ row_weight, float* __restrict__ row_floor,
+    const typename S::T* __restrict__ zi, int64_t zi_stride, const typename S::T* __restrict__ zf,
+    int64_t zf_stride, const float* __restrict__ bias_i, const float* __restrict__ bias_f, float cap,
+    float* __restrict__ maximum, const int* __restrict__ query_start_loc,
+    const int* __restrict__ context_lens, const int* __restrict__ state_slots, int heads) {
+  __shared__ double wave_a[16];
+  __shared__ float wave_b[16];
+  __shared__ float m_lds[1025];
+  const int h = blockIdx.x, b = blockIdx.y;
+  const int t_begin = query_start_loc[b], t_end = query_start_loc[b + 1];
+  const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6;
+  float* m_state = maximum + (int64_t)state_slots[b] * heads + h;
+  float m0 = context_lens[b] > 0 ? *m_state : 0.f;      // every thread holds the maximum before the stretch
+  for (int t0 = t_begin; t0 < t_end; t0 += blockDim.x) {
+    const int t = t0 + tid, n = min((int)blockDim.x, t_end - t0);
+    const bool live = tid < n;
+    float i = -INFINITY, f = 0.f;                       // a row behind the end changes nothing
+    if (live) {
+      i = capped(S::to_f32(zi[(int64_t)t * zi_stride + h]) + bias_i[h], cap);
+      const float c = capped(S::to_f32(zf[(int64_t)t * zf_stride + h]) + bias_f[h], cap);
+      f = -(fmaxf(-c, 0.f) + log1pf(expf(-fabsf(c))));
+    }
+    double a = f;                                       // m -> max(a + m, best) over the rows so far
+    float best = i;
+#pragma unroll
+    for (int s = 1; s < 64; s <<= 1) {
+      const double oa = __shfl_up(a, s, 64);
+      const float ob = __shfl_up(best, s, 64);
+      if (lane >= s) {
+        best = fmaxf((float)(a + (double)ob), best);
+        a += oa;
+      }
+    }
+    if (lane == 63) {
+      wave_a[w] = a;
+      wave_b[w] = best;
+    }
+    __syncthreads();
+    float m_in = m0;
+    for (int o = 0; o < w; ++o) m_in = fmaxf((float)(wave_a[o] + (double)m_in), wave_b[o]);
+    const float m = fmaxf((float)(a + (double)m_in), best);
+    m_lds[tid + 1] = m;
+    if (tid == 0) m_lds[0] = m0;
+    __syncthreads();
+    if (live) {
+      const int64_t at = (int64_t)t * heads + h;
+      row_log[at] = (float)((double)f + (double)m_lds[tid] - (double)m);
+      row_weight[at] = expf(i - m);
+      row_floor[at] = expf(-m);
+    }
+    m0 = m_lds[n];
+    __syncthreads();
+  }
+  if (tid == 0) *m_state = m0;
+}
+
+// Parts of up to 256 numbers, 16-byte aligned: LANES lanes share a part, four numbers each, and norm it
+// with lane sums; 256 / LANES parts per workgroup.
+template <class S, int LANES>
+__global__ __launch_bounds__(256) void gated_small_part_norm_kernel(
+    typename S::T* __restrict__ out, int64_t out_stride, const float* __restrict__ o,
+    const float* __restrict__ weight, const typename S::T* __restrict__ gate, int64_t gate_stride,
+    int gate_act, int gate_first, float eps, int groups, int part, int64_t parts,
+    const float* __restrict__ part_scale) {
+  const int64_t p = (int64_t)blockIdx.x * (256 / LANES) + threadIdx.x / LANES;
+  const int c = 4 * (threadIdx.x % LANES);
+  if (p >= parts) return;                               // whole groups of lanes
+  const int64_t t = p / groups;
+  const int first = (int)(p - t * groups) * part;
+  const bool mine = c < part;
+  f32x4 x = {0.f, 0.f, 0.f, 0.f}, z = x, wv = x;
+  if (mine) {
+    x = *reinterpret_cast<const f32x4*>(o + p * part + c);
+    wv = *reinterpret_cast<const f32x4*>(weight + first + c);
+    const typename S::T* gr = gate + t * gate_stride + first + c;
+    if constexpr (sizeof(typename S::T) == 2) {
+      const u32x2 zz = *reinterpret_cast<const u32x2*>(gr);
+      z = f32x4{lo16<S>(zz[0]), hi16<S>(zz[0]), lo16<S>(zz[1]), hi16<S>(zz[1])};
+    } else {
+      z = *reinterpret_cast<const f32x4*>(gr);
+    }
+  }
+  const float ps = part_scale != nullptr ? part_scale[p] : 1.f;
+  float ss = 0.f;
+#pragma unroll
+  for (int e = 0; e < 4; ++e) {
+    z[e] = gate_act == VLA_GATE_SILU ? silu_f(z[e]) : 1.f / (1.f + expf(-z[e]));
+    x[e] *= ps;
+    if (gate_first) x[e] *= z[e];
+    ss += x[e] * x[e];
+  }
+#pragma unroll
+  for (int m = 1; m < LANES; m <<= 1) ss += __shfl_xor(ss, m, 64);
+  const float inv = 1.f / sqrtf(ss / (float)part + eps);
+  if (!mine) return;
+  float r[4];
+#pragma unroll
+  for (int e = 0; e < 4; ++e) r[e] = x[e] * inv * wv[e] * (gate_first ? 1.f : z[e]);
+  typename S::T* dst = out + t * out_stride + first + c;
+  if constexpr (sizeof(typename S::T) == 2)
+    *reinterpret_cast<u32x2*>(dst) = u32x2{pack16<S>(r[0], r[1]), pack16<S>(r[2], r[3])};
+  else
+    *reinterpret_cast<f32x4*>(dst) = f32x4{r[0], r[1], r[2], r[3]};
 }
 
 // One workgroup per (token, part).  A thread keeps up to four vectors of its part in registers.
@@ -587,7 +785,7 @@ template <class S, int VW>
 __global__ __launch_bounds__(256) void gated_group_rms_norm_kernel(
     typename S::T* __restrict__ out, int64_t out_stride, const float* __restrict__ o,
     const float* __restrict__ weight, const typename S::T* __restrict__ gate, int64_t gate_stride,
-    int gate_act, int gate_first, float eps, int n, int part) {
+    int gate_act, int gate_first, float eps, int n, int part, const float* __restrict__ part_scale) {
   __shared__ float red[16];
   constexpr int KEEP = 16 / VW;
   const int64_t t = blockIdx.x;
@@ -597,6 +795,7 @@ __global__ __launch_bounds__(256) void gated_group_rms_norm_kernel(
   typename S::T* out_row = out + t * out_stride + first;
   const float* wrow = weight + first;
   const int step = blockDim.x * VW;
+  const float ps = part_scale != nullptr ? part_scale[t * gridDim.y + blockIdx.y] : 1.f;
   auto gated = [&](float z) { return gate_act == VLA_GATE_SILU ? silu_f(z) : 1.f / (1.f + expf(-z)); };
   auto read = [&](int c, float (&u)[VW], float (&f)[VW]) {     // the value to norm, and the factor after it
     float x[VW], z[VW];
@@ -622,7 +821,7 @@ __global__ __launch_bounds__(256) void gated_group_rms_norm_kernel(
 #pragma unroll
     for (int e = 0; e < VW; ++e) {
       const float gv = gated(z[e]);
-      u[e] = gate_first ? x[e] * gv : x[e];
+      u[e] = x[e] * ps * (gate_first ? gv : 1.f);
       f[e] = gate_first ? 1.f : gv;
     }
   };
@@ -689,8 +888,7 @@ int launch_blocks(const DecayScan& a, int pieces, hipStream_t stream) {
   if (a.piece_rows > 0) {
     const int rc = launch_block<DB, WAVES, KIND, true>(a, pieces, stream);
     if (rc != VLA_OK) return rc;
-    const int64_t size = (int64_t)a.dim * a.vdim;
-    decay_chain_kernel<<<dim3((unsigned)((size + 255) / 256), a.heads, a.num_seqs), 256, 0, stream>>>(a);
+    decay_chain_kernel<<<dim3((unsigned)((a.head_size + 255) / 256), a.heads, a.num_seqs), 256, 0, stream>>>(a);
     VLA_SEQ_HIP_CHECK(hipGetLastError());
   }
   return launch_block<DB, WAVES, KIND, false>(a, pieces, stream);
@@ -724,9 +922,9 @@ using namespace vla;
 using namespace vla::seq;
 
 extern "C" int64_t vla_seq_decay_scan_scratch_floats(int num_tokens, int num_seqs, int max_query_len,
-                                                     int heads, int dim, int vdim) {
+                                                     int heads, int dim, int vdim, int normalizer) {
   if (!cuts_runs(max_query_len, dim)) return 0;
-  return piece_slots(num_tokens, num_seqs) * heads * ((int64_t)dim * vdim + 1);
+  return piece_slots(num_tokens, num_seqs) * heads * ((int64_t)dim * (vdim + (normalizer ? 1 : 0)) + 1);
 }
 
 extern "C" int vla_seq_set_decay_scan_kernel(int mode) {
@@ -738,7 +936,9 @@ extern "C" int vla_seq_set_decay_scan_kernel(int mode) {
 extern "C" int vla_seq_decay_scan(float* o, const void* q, int64_t q_stride, const void* k,
                                   int64_t k_stride, const void* v, int64_t v_stride, const void* dt,
                                   int64_t dt_stride, const float* dt_bias, const float* a_log,
-                                  const float* log_decay, const float* skip, float* state,
+                                  const float* log_decay, const float* skip, const float* row_log,
+                                  const float* row_weight, const float* row_floor,
+                                  float* norm_scale, float norm_eps, float q_scale, float* state,
                                   const int* query_start_loc, const int* context_lens,
                                   const int* state_slots, int num_tokens, int num_seqs,
                                   int num_slots, int max_query_len, int heads, int groups, int dim,
@@ -750,9 +950,10 @@ extern "C" int vla_seq_decay_scan(float* o, const void* q, int64_t q_stride, con
       heads <= 0 || groups <= 0 || heads % groups != 0 || dim <= 0 || vdim <= 0 ||
       q_stride < (int64_t)groups * dim || k_stride < (int64_t)groups * dim ||
       v_stride < (int64_t)heads * vdim || (act != VLA_ACT_NONE && act != VLA_ACT_SILU) ||
-      (dt ? (!dt_bias || !a_log || dt_stride < heads) : !log_decay))
+      (row_log ? !row_weight : dt ? (!dt_bias || !a_log || dt_stride < heads) : !log_decay) ||
+      (norm_scale && !row_floor))
     return VLA_ERR_ARG;
-  if (dim > 1024 || vdim > 256) return VLA_ERR_HEAD_SIZE;
+  if (dim > 1024 || vdim > (vdim % 4 == 0 ? 1024 : 256)) return VLA_ERR_HEAD_SIZE;
   if (dtype != VLA_F16 && dtype != VLA_BF16 && dtype != VLA_F32) return VLA_ERR_DTYPE;
   hipStream_t st = (hipStream_t)stream;
   const int elem = dtype == VLA_F32 ? 4 : 2;
@@ -773,6 +974,13 @@ extern "C" int vla_seq_decay_scan(float* o, const void* q, int64_t q_stride, con
   a.a_log = a_log;
   a.log_decay = log_decay;
   a.skip = skip;
+  a.row_log = row_log;
+  a.row_weight = row_weight;
+  a.row_floor = row_floor;
+  a.norm_scale = norm_scale;
+  a.norm_eps = norm_eps;
+  a.q_scale = q_scale;
+  a.head_size = (int64_t)dim * (vdim + (norm_scale ? 1 : 0));
   a.state = state;
   a.query_start_loc = query_start_loc;
   a.context_lens = context_lens;
@@ -794,20 +1002,21 @@ extern "C" int vla_seq_decay_scan(float* o, const void* q, int64_t q_stride, con
   int pieces = num_seqs;
   if (a.mode != 1 && cuts_runs(max_query_len, dim)) {
     const int64_t slots = piece_slots(num_tokens, num_seqs);
-    const int64_t need = slots * heads * ((int64_t)dim * vdim + 1);
+    const int64_t need = slots * heads * (a.head_size + 1);
     if (!scratch || scratch_floats < need || slots > 65535) return VLA_ERR_ARG;
     a.piece_rows = VLA_DECAY_SCAN_PIECE;
     a.piece_state = scratch;
-    a.piece_decay = scratch + slots * heads * ((int64_t)dim * vdim);
+    a.piece_decay = scratch + slots * heads * a.head_size;
     pieces = (int)slots;
   }
   // a step of several sequences may hold runs of both kinds: each launch skips the other's sequences
   const bool steps = a.mode == 1 || (a.mode == 0 && (max_query_len <= kStepRows || num_seqs > 1));
   const bool blocks = a.mode == 2 || (a.mode == 0 && max_query_len > kStepRows);
   if (steps) {
-    const int vw = vdim % 4 == 0 && ((uintptr_t)state % 16) == 0 ? 4 : 1;
+    const int vw = vdim % 4 == 0 && a.head_size % 4 == 0 && ((uintptr_t)state % 16) == 0 ? 4 : 1;
     const int cols = (vdim + vw - 1) / vw, groups_of_rows = 256 / cols;
-    const size_t lds = sizeof(float) * (2 * (size_t)dim + vdim + (size_t)groups_of_rows * vdim);
+    if (groups_of_rows < 1) return VLA_ERR_HEAD_SIZE;
+    const size_t lds = sizeof(float) * (2 * (size_t)dim + vdim + (size_t)groups_of_rows * vdim + 4);
     const dim3 grid(heads, num_seqs);
     if (vw == 4)
       decay_step_kernel<4><<<grid, 256, lds, st>>>(a);
@@ -825,7 +1034,7 @@ extern "C" int vla_seq_gated_group_rms_norm(void* out, int64_t out_stride, const
                                             const float* weight, const void* gate,
                                             int64_t gate_stride, int gate_act, int gate_first,
                                             int groups, float eps, int num_tokens, int n, int dtype,
-                                            void* stream) {
+                                            const float* part_scale, void* stream) {
   if (num_tokens == 0) return VLA_OK;
   if (!out || !o || !weight || !gate || num_tokens < 0 || n <= 0 || groups <= 0 || n % groups != 0 ||
       groups > 65535 || out_stride < n || gate_stride < n ||
@@ -840,12 +1049,56 @@ extern "C" int vla_seq_gated_group_rms_norm(void* out, int64_t out_stride, const
     const int64_t bytes = 4 * sizeof(T);
     const bool vec = part % 4 == 0 && ((uintptr_t)o % 16) == 0 && (uintptr_t)gate % bytes == 0 &&
                      (uintptr_t)out % bytes == 0 && gate_stride % 4 == 0 && out_stride % 4 == 0;
+    if (vec && groups > 1 && part <= 256 && ((uintptr_t)weight % 16) == 0) {
+      const int64_t parts = (int64_t)num_tokens * groups;
+      auto small = [&](auto kernel, int lanes) {
+        const int per = 256 / lanes;
+        kernel<<<(unsigned)((parts + per - 1) / per), 256, 0, (hipStream_t)stream>>>(
+            (T*)out, out_stride, o, weight, (const T*)gate, gate_stride, gate_act, gate_first, eps, groups, part,
+            parts, part_scale);
+      };
+      if (part <= 64)
+        small(gated_small_part_norm_kernel<S, 16>, 16);
+      else if (part <= 128)
+        small(gated_small_part_norm_kernel<S, 32>, 32);
+      else
+        small(gated_small_part_norm_kernel<S, 64>, 64);
+      VLA_SEQ_HIP_CHECK(hipGetLastError());
+      return (int)VLA_OK;
+    }
     if (vec)
       gated_group_rms_norm_kernel<S, 4><<<grid, threads, 0, (hipStream_t)stream>>>(
-          (T*)out, out_stride, o, weight, (const T*)gate, gate_stride, gate_act, gate_first, eps, n, part);
+          (T*)out, out_stride, o, weight, (const T*)gate, gate_stride, gate_act, gate_first, eps, n, part,
+          part_scale);
     else
       gated_group_rms_norm_kernel<S, 1><<<grid, threads, 0, (hipStream_t)stream>>>(
-          (T*)out, out_stride, o, weight, (const T*)gate, gate_stride, gate_act, gate_first, eps, n, part);
+          (T*)out, out_stride, o, weight, (const T*)gate, gate_stride, gate_act, gate_first, eps, n, part,
+          part_scale);
+    VLA_SEQ_HIP_CHECK(hipGetLastError());
+    return (int)VLA_OK;
+  });
+}
+
+extern "C" int vla_seq_matrix_memory_gates(float* row_log, float* row_weight, float* row_floor,
+                                           const void* zi, int64_t zi_stride, const void* zf,
+                                           int64_t zf_stride, const float* bias_i,
+                                           const float* bias_f, float cap, float* maximum,
+                                           const int* query_start_loc, const int* context_lens,
+                                           const int* state_slots, int num_seqs, int num_slots,
+                                           int max_query_len, int heads, int dtype, void* stream) {
+  if (num_seqs == 0) return VLA_OK;
+  if (!row_log || !row_weight || !row_floor || !zi || !zf || !bias_i || !bias_f || !maximum ||
+      !query_start_loc || !context_lens || !state_slots || num_seqs < 0 || num_seqs > 65535 ||
+      num_slots <= 0 || max_query_len <= 0 || heads <= 0 || zi_stride < heads || zf_stride < heads ||
+      !(cap > 0.f))
+    return VLA_ERR_ARG;
+  const int threads = max_query_len <= 64 ? 64 : max_query_len <= 256 ? 256 : 1024;
+  return with_dtype(dtype, [&](auto s) {
+    using S = decltype(s);
+    using T = typename S::T;
+    matrix_memory_gates_kernel<S><<<dim3(heads, num_seqs), threads, 0, (hipStream_t)stream>>>(
+        row_log, row_weight, row_floor, (const T*)zi, zi_stride, (const T*)zf, zf_stride, bias_i, bias_f, cap,
+        maximum, query_start_loc, context_lens, state_slots, heads);
     VLA_SEQ_HIP_CHECK(hipGetLastError());
     return VLA_OK;
   });

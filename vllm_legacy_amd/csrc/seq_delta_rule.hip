@@ -31,36 +31,6 @@ namespace {
 constexpr int kMaxChunk = 32;
 constexpr int kMaxSplit = 16;
 
-// v + the value another lane holds, the lanes paired by a DPP pattern (no LDS round trip)
-template <int CTRL>
-__device__ __forceinline__ float dpp_add(float v) {
-  const int other = __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), CTRL, 0xf, 0xf, false);
-  return v + __builtin_bit_cast(float, other);
-}
-
-// the sum over each aligned group of `split` lanes (1, 2, 4, 8 or 16), in every lane of the group:
-// neighbours, pairs of a quad, the mirrored half of eight, the mirrored half of sixteen
-__device__ __forceinline__ void group_sums(float& a, float& b, int split) {
-  if (split > 1) {
-    a = dpp_add<0xB1>(a);      // quad_perm [1, 0, 3, 2]
-    b = dpp_add<0xB1>(b);
-  }
-  if (split > 2) {
-    a = dpp_add<0x4E>(a);      // quad_perm [2, 3, 0, 1]
-    b = dpp_add<0x4E>(b);
-  }
-  if (split > 4) {
-    a = dpp_add<0x141>(a);     // row_half_mirror: lane i of eight with lane 7 - i
-    b = dpp_add<0x141>(b);
-  }
-  if (split > 8) {
-    a = dpp_add<0x140>(a);     // row_mirror: lane i of sixteen with lane 15 - i
-    b = dpp_add<0x140>(b);
-  }
-}
-
-__device__ __forceinline__ float softplusf(float z) { return z > 20.f ? z : log1pf(expf(z)); }
-
 template <class SI>
 struct DeltaRows {
   const typename SI::T* q;

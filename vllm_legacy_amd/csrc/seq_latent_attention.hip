@@ -11,8 +11,9 @@
 // attention kernels then read every query row's keys from the cache, so prompts, portions of
 // prompts and decode steps are one case.  An optional window keeps 0 <= p - j < window; an optional
 // gate multiplies a head's sums by the sigmoid of one number per (token, head) (the head's
-// up-projection that follows is linear, so the gate may stand on either side of it).  Angles, norms,
-// scores, softmax and the weighted sum are fp32.
+// up-projection that follows is linear, so the gate may stand on either side of it); optional sinks
+// add exp(sink_h) to a head's denominator: the softmax starts from maximum = sink, sum = 1 instead of
+// from nothing.  Angles, norms, scores, softmax and the weighted sum are fp32.
 //
 // latent_attention_kernel: one wave per (token, head), any dtype, rank up to 1024.  A tile is 64
 // keys: lane j scores key j against the query held in LDS, the wave reduces max / sum (online
@@ -99,7 +100,7 @@ __global__ __launch_bounds__(kWave* kHeadsPerGroup) void latent_attention_kernel
     LatentQuery<S> q, const typename S::T* __restrict__ cache, const int* __restrict__ block_tables,
     int max_blocks, const int* __restrict__ token_seq, const int64_t* __restrict__ positions,
     int heads, int rank, int rot, int block_size, int num_blocks, float scale, int window,
-    const typename S::T* __restrict__ gate, int64_t gate_stride) {
+    const typename S::T* __restrict__ gate, int64_t gate_stride, const float* __restrict__ sinks) {
   extern __shared__ float lds[];
   const int width = rank + rot;
   const int lane = threadIdx.x & 63, w = threadIdx.x >> 6;
@@ -125,7 +126,7 @@ __global__ __launch_bounds__(kWave* kHeadsPerGroup) void latent_attention_kernel
   float acc[kAccum];
 #pragma unroll
   for (int c = 0; c < kAccum; ++c) acc[c] = 0.f;
-  float m = -INFINITY, l = 0.f;
+  float m = sinks != nullptr ? sinks[h] : -INFINITY, l = sinks != nullptr ? 1.f : 0.f;
   const int lo = window > 0 ? max(0, p - window + 1) : 0;
   for (int j0 = lo; j0 <= p; j0 += kWave) {
     const int j = j0 + lane;
@@ -226,7 +227,8 @@ __global__ __launch_bounds__(256) void latent_attention_tile_kernel(
     int max_blocks, const int* __restrict__ query_start_loc, const int* __restrict__ context_lens,
     int heads, int rank, int rot, int block_size, int num_blocks, float scale, int hb, int tb,
     int key_splits, float* __restrict__ part_o, float* __restrict__ part_ml, int num_tokens,
-    int window, const typename S::T* __restrict__ gate, int64_t gate_stride) {
+    int window, const typename S::T* __restrict__ gate, int64_t gate_stride,
+    const float* __restrict__ sinks) {
   using T = typename S::T;
   using M = LatentMfma<S>;
   constexpr int WP = 2 * VBW + 2;                      // 16-byte pieces of a tile a thread stages
@@ -282,6 +284,10 @@ __global__ __launch_bounds__(256) void latent_attention_tile_kernel(
 #pragma unroll
     for (int i = 0; i < 16; ++i) o[n][i] = 0.f;
   float m = -INFINITY, l = 0.f;
+  if (sinks != nullptr && split == 0 && my_row) {      // once per row: in the first share, in one lane half's sum
+    m = sinks[h0 + my_head] * 1.4426950408889634f;
+    l = hf == 0 ? 1.f : 0.f;
+  }
 
   // threads 0 .. 31 look the rows of a tile up: the block id is read one step before it is used
   auto load_block = [&](int j0) {
@@ -517,7 +523,7 @@ int launch_latent_tiles(dim3 grid, size_t lds, hipStream_t stream, typename S::T
                         const int* qsl, const int* ctx, int heads, int rank, int rot, int block_size,
                         int num_blocks, float scale, int hb, int tb, int key_splits, float* part_o,
                         float* part_ml, int num_tokens, int window, const typename S::T* gate,
-                        int64_t gate_stride) {
+                        int64_t gate_stride, const float* sinks) {
   static std::atomic<size_t> allowed{64 * 1024};   // raised once per kernel, not per launch
   if (lds > allowed.load(std::memory_order_relaxed)) {
     VLA_SEQ_HIP_CHECK(hipFuncSetAttribute(
@@ -528,7 +534,7 @@ int launch_latent_tiles(dim3 grid, size_t lds, hipStream_t stream, typename S::T
   latent_attention_tile_kernel<S, VBW><<<grid, 256, lds, stream>>>(
       out, out_token_stride, out_head_stride, q, cache, block_tables, max_blocks, qsl, ctx, heads,
       rank, rot, block_size, num_blocks, scale, hb, tb, key_splits, part_o, part_ml, num_tokens,
-      window, gate, gate_stride);
+      window, gate, gate_stride, sinks);
   VLA_SEQ_HIP_CHECK(hipGetLastError());
   if (key_splits > 1) {
     latent_merge_kernel<S><<<(unsigned)((int64_t)num_tokens * heads), 256, 0, stream>>>(
@@ -581,7 +587,8 @@ extern "C" int vla_seq_latent_attention(void* out, int64_t out_token_stride, int
                                         const int* token_seq, const int64_t* positions,
                                         int num_tokens, int heads, int rank, int rot, int block_size,
                                         int num_blocks, float scale, int dtype, int window,
-                                        const void* gate, int64_t gate_stride, void* stream) {
+                                        const void* gate, int64_t gate_stride, const float* sinks,
+                                        void* stream) {
   if (num_tokens == 0) return VLA_OK;
   if (gate && gate_stride < heads) return VLA_ERR_ARG;
   if (!out || !q_lat || (rot > 0 && !q_rot) || !cache || !block_tables || !token_seq || !positions ||
@@ -599,7 +606,7 @@ extern "C" int vla_seq_latent_attention(void* out, int64_t out_token_stride, int
     latent_attention_kernel<S><<<grid, kWave * kHeadsPerGroup, lds, (hipStream_t)stream>>>(
         (T*)out, out_token_stride, out_head_stride, q, (const T*)cache, block_tables, max_blocks,
         token_seq, positions, heads, rank, rot, block_size, num_blocks, scale, window, (const T*)gate,
-        gate_stride);
+        gate_stride, sinks);
     VLA_SEQ_HIP_CHECK(hipGetLastError());
     return VLA_OK;
   });
@@ -628,7 +635,8 @@ extern "C" int vla_seq_latent_attention_tiles(
     int64_t rot_head_stride, const void* cache, const int* block_tables, int max_blocks,
     const int* query_start_loc, const int* context_lens, int num_seqs, int max_query_len, int heads,
     int rank, int rot, int block_size, int num_blocks, float scale, int key_splits, float* scratch,
-    int num_tokens, int dtype, int window, const void* gate, int64_t gate_stride, void* stream) {
+    int num_tokens, int dtype, int window, const void* gate, int64_t gate_stride, const float* sinks,
+    void* stream) {
   if (num_seqs == 0 || max_query_len == 0) return VLA_OK;
   if (gate && gate_stride < heads) return VLA_ERR_ARG;
   if (!out || !q_lat || (rot > 0 && !q_rot) || !cache || !block_tables || !query_start_loc ||
@@ -663,7 +671,7 @@ extern "C" int vla_seq_latent_attention_tiles(
                                      out_head_stride, q, (const T*)cache, block_tables, max_blocks, \
                                      query_start_loc, context_lens, heads, rank, rot, block_size,   \
                                      num_blocks, scale, hb, tb, key_splits, part_o, part_ml,        \
-                                     num_tokens, window, (const T*)gate, gate_stride);
+                                     num_tokens, window, (const T*)gate, gate_stride, sinks);
     switch (vbw) {
       VLA_LATENT_CASE(1)
       VLA_LATENT_CASE(2)

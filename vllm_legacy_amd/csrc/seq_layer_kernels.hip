@@ -114,6 +114,117 @@ __global__ __launch_bounds__(kThreads) void residual_norms_kernel(
     out[base + c] = SO::from_f32(x[base + c] * inv * pre_w[c]);
 }
 
+// The stream's update where a layer's branches all read the stream of the layer's start, and the norms of
+// its readers: x += sum of up to three scaled rows and of a token's expert rows, then one root mean
+// square and a copy per reader with its own weight.  VW values per access; a thread keeps up to 16 of
+// its row between the reduction and the writes.
+constexpr int kMaxTerms = 3;
+constexpr int kMaxReaders = 2;
+struct BranchSum {
+  float* x;
+  const float* term[kMaxTerms];
+  float scale[kMaxTerms];
+  const float* expert_rows;         // fp32 [rows, width]
+  const int* pair_row;              // [T, top]
+  const float* pair_weight;         // [T, top]
+  void* out[kMaxReaders];
+  const float* weight[kMaxReaders];
+  float eps;
+  int top, width;
+};
+
+template <int VW>
+struct RowVec {
+  float v[VW];
+};
+template <int VW>
+__device__ __forceinline__ RowVec<VW> read_row(const float* p) {
+  RowVec<VW> r;
+  if constexpr (VW == 4) {
+    const f32x4 q = *reinterpret_cast<const f32x4*>(p);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) r.v[e] = q[e];
+  } else {
+    r.v[0] = *p;
+  }
+  return r;
+}
+
+template <class SO, int VW>
+__global__ __launch_bounds__(kThreads) void branch_sum_norms_kernel(BranchSum a) {
+  constexpr int KEEP = 16 / VW;
+  __shared__ float red[16];
+  const int64_t t = blockIdx.x, base = t * a.width;
+  const int step = kThreads * VW;
+  const bool writes = a.term[0] != nullptr || a.expert_rows != nullptr;
+  float ss = 0.f;
+  auto update = [&](int c) {
+    RowVec<VW> x = read_row<VW>(a.x + base + c);
+#pragma unroll
+    for (int i = 0; i < kMaxTerms; ++i)
+      if (a.term[i] != nullptr) {
+        const RowVec<VW> y = read_row<VW>(a.term[i] + base + c);
+#pragma unroll
+        for (int e = 0; e < VW; ++e) x.v[e] += a.scale[i] * y.v[e];
+      }
+    if (a.expert_rows != nullptr) {
+      RowVec<VW> sum = {};
+      for (int k = 0; k < a.top; ++k) {
+        const int row = a.pair_row[t * a.top + k];
+        if (row < 0) continue;
+        const float wk = a.pair_weight[t * a.top + k];
+        const RowVec<VW> y = read_row<VW>(a.expert_rows + (int64_t)row * a.width + c);
+#pragma unroll
+        for (int e = 0; e < VW; ++e) sum.v[e] += wk * y.v[e];
+      }
+#pragma unroll
+      for (int e = 0; e < VW; ++e) x.v[e] += sum.v[e];
+    }
+    if (writes) {
+      if constexpr (VW == 4)
+        *reinterpret_cast<f32x4*>(a.x + base + c) = f32x4{x.v[0], x.v[1], x.v[2], x.v[3]};
+      else
+        a.x[base + c] = x.v[0];
+    }
+#pragma unroll
+    for (int e = 0; e < VW; ++e) ss += x.v[e] * x.v[e];
+    return x;
+  };
+  RowVec<VW> keep[KEEP];
+#pragma unroll
+  for (int i = 0; i < KEEP; ++i) {
+    const int c = threadIdx.x * VW + i * step;
+    if (c < a.width) keep[i] = update(c);
+  }
+  for (int c = threadIdx.x * VW + KEEP * step; c < a.width; c += step) update(c);
+  if (a.out[0] == nullptr) return;
+  ss = block_sum(ss, red);
+  const float inv = 1.f / sqrtf(ss / (float)a.width + a.eps);
+  auto write = [&](int c, const RowVec<VW>& x) {
+#pragma unroll
+    for (int o = 0; o < kMaxReaders; ++o)
+      if (a.out[o] != nullptr) {
+        const RowVec<VW> w = read_row<VW>(a.weight[o] + c);
+        typename SO::T* dst = (typename SO::T*)a.out[o] + base + c;
+        float r[VW];
+#pragma unroll
+        for (int e = 0; e < VW; ++e) r[e] = x.v[e] * inv * w.v[e];
+        if constexpr (VW == 4 && sizeof(typename SO::T) == 2) {
+          *reinterpret_cast<u32x2*>(dst) = u32x2{pack16<SO>(r[0], r[1]), pack16<SO>(r[2], r[3])};
+        } else {
+#pragma unroll
+          for (int e = 0; e < VW; ++e) dst[e] = SO::from_f32(r[e]);
+        }
+      }
+  };
+#pragma unroll
+  for (int i = 0; i < KEEP; ++i) {
+    const int c = threadIdx.x * VW + i * step;
+    if (c < a.width) write(c, keep[i]);
+  }
+  for (int c = threadIdx.x * VW + KEEP * step; c < a.width; c += step) write(c, read_row<VW>(a.x + base + c));
+}
+
 // out[t] = h[t] + sum_d w[:, taps - 1 - d] * h at position p - d; rows of earlier steps come from
 // the state slot, positions before the sequence's start are zeros.
 template <class S>
@@ -265,6 +376,35 @@ extern "C" int vla_seq_residual_norms(float* x, const void* y, int64_t y_stride,
       residual_norms_kernel<SY, SO, false><<<num_tokens, kThreads, 0, (hipStream_t)stream>>>(
           x, (const TY*)y, y_stride, y_bias, post_weight, layer_scale, add_row, (typename SO::T*)out,
           pre_weight, eps, width, y_scale, nullptr, 0, nullptr);
+    VLA_SEQ_HIP_CHECK(hipGetLastError());
+    return VLA_OK;
+  });
+}
+
+extern "C" int vla_seq_branch_sum_norms(float* x, const float* y0, float s0, const float* y1, float s1,
+                                        const float* y2, float s2, const float* expert_rows,
+                                        const int* pair_row, const float* pair_weight, int top,
+                                        void* out0, const float* weight0, void* out1,
+                                        const float* weight1, float eps, int num_tokens, int width,
+                                        int out_dtype, void* stream) {
+  if (num_tokens == 0) return VLA_OK;
+  if (!x || num_tokens < 0 || width <= 0 || (!y0 && (y1 || y2)) || (!out0 && out1) || (out0 && !weight0) ||
+      (out1 && !weight1) || (expert_rows && (!pair_row || !pair_weight || top <= 0)))
+    return VLA_ERR_ARG;
+  const BranchSum a{x, {y0, y1, y2}, {s0, s1, s2}, expert_rows, pair_row, pair_weight, {out0, out1},
+                    {weight0, weight1}, eps, top, width};
+  return with_dtype(out0 ? out_dtype : VLA_F32, [&](auto so) {
+    using SO = decltype(so);
+    const size_t out_bytes = 4 * sizeof(typename SO::T);
+    bool vec = width % 4 == 0;
+    for (const void* p : {(const void*)x, (const void*)y0, (const void*)y1, (const void*)y2,
+                          (const void*)expert_rows, (const void*)weight0, (const void*)weight1})
+      vec = vec && (uintptr_t)p % 16 == 0;
+    for (const void* p : {(const void*)out0, (const void*)out1}) vec = vec && (uintptr_t)p % out_bytes == 0;
+    if (vec)
+      branch_sum_norms_kernel<SO, 4><<<num_tokens, kThreads, 0, (hipStream_t)stream>>>(a);
+    else
+      branch_sum_norms_kernel<SO, 1><<<num_tokens, kThreads, 0, (hipStream_t)stream>>>(a);
     VLA_SEQ_HIP_CHECK(hipGetLastError());
     return VLA_OK;
   });

@@ -1,8 +1,9 @@
 // Mixture-of-experts feed-forward in the activation dtype (no quantization), routed on the device
 // without a host synchronisation:
 //   moe_route      per token: router logits in fp32 (plus a bias), softmax over all experts or the
-//                  sigmoid of each logit, choice by score plus a per-expert correction, weights = chosen
-//                  scores, renormalized or as they are; also the sigmoid gate of a shared expert
+//                  sigmoid of each logit, choice by score plus a per-expert correction (among the best
+//                  groups of neighbouring experts, where there are groups), weights = chosen scores,
+//                  renormalized or as they are, times a scale; also the sigmoid gate of a shared expert
 //   moe_plan       groups the (token, choice) pairs by expert into row tiles of kTile rows (groups
 //                  are padded to whole tiles, so a tile belongs to one expert)
 //   grouped_linear out[row] = act(W_e a[row] * scale[row]) for the rows of every tile, W_e the tile's expert;
@@ -43,8 +44,11 @@ __global__ __launch_bounds__(256) void moe_route_kernel(
     const float* __restrict__ logits, int64_t logits_stride, const float* __restrict__ bias,
     const float* __restrict__ correction,
     const float* __restrict__ shared_gate_w, int* __restrict__ experts, float* __restrict__ weights,
-    float* __restrict__ shared_gate, int width, int routed, int top, int score, int renormalize) {
+    float* __restrict__ shared_gate, int width, int routed, int top, int score, int renormalize,
+    int groups, int keep_groups, float weight_scale) {
   __shared__ float z[kMaxRouted + 1];
+  __shared__ float group_best[kMaxRouted];
+  __shared__ int group_open[kMaxRouted];
   const int t = blockIdx.x, lane = threadIdx.x & 63, w = threadIdx.x >> 6;
   const bool gated = shared_gate != nullptr;
   const int rows = routed + (gated ? 1 : 0);
@@ -96,6 +100,33 @@ __global__ __launch_bounds__(256) void moe_route_kernel(
     const int n = lane + i * kWave;
     choice[i] = n < routed ? s[i] + (correction != nullptr ? correction[n] : 0.f) : -INFINITY;
   }
+  if (keep_groups < groups) {
+    // a group's score is its best choice; only experts of the keep_groups best groups stay
+    const int size = routed / groups;
+    wave_sync();
+#pragma unroll
+    for (int i = 0; i < PER; ++i)
+      if (lane + i * kWave < routed) z[lane + i * kWave] = choice[i];
+    wave_sync();
+    for (int g = lane; g < groups; g += kWave) {
+      float best = -INFINITY;
+      for (int n = 0; n < size; ++n) best = fmaxf(best, z[g * size + n]);
+      group_best[g] = best;
+    }
+    wave_sync();
+    for (int g = lane; g < groups; g += kWave) {
+      int ahead = 0;                 // groups that go first: better ones, and equal ones with a lower index
+      for (int o = 0; o < groups; ++o)
+        ahead += group_best[o] > group_best[g] || (group_best[o] == group_best[g] && o < g) ? 1 : 0;
+      group_open[g] = ahead < keep_groups;
+    }
+    wave_sync();
+#pragma unroll
+    for (int i = 0; i < PER; ++i) {
+      const int n = lane + i * kWave;
+      if (n < routed && !group_open[n / size]) choice[i] = -INFINITY;
+    }
+  }
   float total = 0.f, mine = 0.f;     // lane k keeps the k-th chosen score
   int mine_e = 0;
   for (int k = 0; k < top; ++k) {
@@ -131,7 +162,7 @@ __global__ __launch_bounds__(256) void moe_route_kernel(
   }
   if (lane < top) {
     experts[(int64_t)t * top + lane] = mine_e;
-    weights[(int64_t)t * top + lane] = renormalize ? mine / (total + 1e-20f) : mine;
+    weights[(int64_t)t * top + lane] = (renormalize ? mine / (total + 1e-20f) : mine) * weight_scale;
   }
 }
 
@@ -526,12 +557,14 @@ extern "C" int vla_seq_moe_route(const void* h, int64_t h_stride, const float* r
                                  const float* logits, int64_t logits_stride, const float* bias,
                                  const float* correction, const float* shared_gate_weight,
                                  int* experts, float* weights, float* shared_gate, int num_tokens,
-                                 int width, int routed, int top, int score, int renormalize, int dtype,
+                                 int width, int routed, int top, int score, int renormalize,
+                                 int groups, int keep_groups, float weight_scale, int dtype,
                                  void* stream) {
   if (num_tokens == 0) return VLA_OK;
   const bool gated = shared_gate != nullptr;
   if (!experts || !weights || num_tokens < 0 || width <= 0 || routed <= 0 || routed > kMaxRouted ||
-      top <= 0 || top > routed || top > kWave ||
+      top <= 0 || top > routed || top > kWave || groups <= 0 || routed % groups != 0 ||
+      keep_groups <= 0 || keep_groups > groups || top > keep_groups * (routed / groups) ||
       (score != VLA_SCORE_SOFTMAX && score != VLA_SCORE_SIGMOID) ||
       (logits ? logits_stride < routed + (gated ? 1 : 0)
               : (!h || !router || h_stride < width || (gated && !shared_gate_weight))))
@@ -540,7 +573,8 @@ extern "C" int vla_seq_moe_route(const void* h, int64_t h_stride, const float* r
     using S = decltype(s);
     moe_route_kernel<S><<<num_tokens, 256, 0, (hipStream_t)stream>>>(
         (const typename S::T*)h, h_stride, router, logits, logits_stride, bias, correction,
-        shared_gate_weight, experts, weights, shared_gate, width, routed, top, score, renormalize);
+        shared_gate_weight, experts, weights, shared_gate, width, routed, top, score, renormalize, groups,
+        keep_groups, weight_scale);
     VLA_SEQ_HIP_CHECK(hipGetLastError());
     return VLA_OK;
   });

@@ -15,6 +15,7 @@ _MODELS: Dict[str, Tuple[str, str, str]] = {
     "Lamosun": ("vllm_legacy_amd.model.lamosun", "LamosunForCausalLM", "LamosunConfig"),
     "Tekezen": ("vllm_legacy_amd.model.tekezen", "TekezenForCausalLM", "TekezenConfig"),
     "Batatar": ("vllm_legacy_amd.model.batatar", "BatatarForCausalLM", "BatatarConfig"),
+    "Dagavik": ("vllm_legacy_amd.model.dagavik", "DagavikForCausalLM", "DagavikConfig"),
     # the synthetic-weight Llama stack behind the engine's model protocol
     "LlamaDecodeStack": ("vllm_legacy_amd.engine.llama_adapter", "PagedLlamaForEngine", "LlamaEngineConfig"),
 }

@@ -4,8 +4,10 @@ Router: z = W_r h (+ a bias) in fp32 over all routed experts, s = softmax(z); th
 with the largest s + correction are chosen and weighted by their s renormalized to sum 1 (without a
 correction: the softmax over the chosen logits).  `score="sigmoid"` takes s = sigmoid(z) of each logit,
 `renormalize=False` the chosen s as they are, and `weight_input=True` lets a choice's weight multiply
-its expert's input instead of its output (the fp32 sums of W_gate h and W_up h are scaled).  The last `identity` routed experts have no
-weights: their output is the token's input.  An expert is W_down act(W_up h), or, `gated`,
+its expert's input instead of its output (the fp32 sums of W_gate h and W_up h are scaled).  With
+`groups` > 1 the experts form that many equal groups of neighbours and only those of the
+`keep_groups` groups with the largest best score can be chosen; `weight_scale` multiplies every
+weight.  The last `identity` routed experts have no weights: their output is the token's input.  An expert is W_down act(W_up h), or, `gated`,
 W_down (act(W_gate h) * W_up h); with act "clamped_glu" the gated form is
 g sigmoid(alpha g) (u + shift), g = min(W_gate h, limit), u = clamp(W_up h, -limit, limit).  An
 optional shared expert runs for every token: plain, multiplied by sigmoid(w_sg . h), or
@@ -43,8 +45,13 @@ class RoutedExperts(nn.Module):
                  dtype=torch.bfloat16, device=None, gated: bool = False, router_bias: bool = False,
                  act_limit: float = 0.0, act_alpha: float = 1.702, act_shift: float = 1.0,
                  shared_gated: bool = False, shared_limit: float = 0.0, score: str = "softmax",
-                 renormalize: bool = True, weight_input: bool = False) -> None:
+                 renormalize: bool = True, weight_input: bool = False, groups: int = 1, keep_groups: int = 1,
+                 weight_scale: float = 1.0) -> None:
         super().__init__()
+        routed = num_experts + num_identity
+        if groups < 1 or routed % groups or not 1 <= keep_groups <= groups or top > keep_groups * (routed // groups):
+            raise ValueError("the groups do not fit the number of routed experts and of choices")
+        self.groups, self.keep_groups, self.weight_scale = int(groups), int(keep_groups), float(weight_scale)
         if score not in ops.MOE_SCORE:
             raise ValueError(f"unknown router score {score!r}")
         if weight_input and num_identity:
@@ -64,7 +71,6 @@ class RoutedExperts(nn.Module):
         self.dtype = dtype
         self.gated = bool(gated)
         self._router_rows = None
-        routed = num_experts + num_identity
 
         def par(shape, dt):
             return nn.Parameter(torch.zeros(shape, dtype=dt, device=device), requires_grad=False)
@@ -127,8 +133,11 @@ class RoutedExperts(nn.Module):
         else:
             ops.gated_act(out, both[:, :ff], both[:, ff:], act)
 
-    def forward(self, h: torch.Tensor) -> torch.Tensor:
-        """h [T, width] in the activation dtype -> fp32 [T, width]."""
+    def rows(self, h: torch.Tensor):
+        """The experts' outputs before their weighted sum: (y fp32 [rows, width], pair_row int32 [T, top],
+        weights fp32 [T, top] or None, shared expert's gate fp32 [T] or None).  A caller that updates a
+        stream with the sum may form it there (_seq_ops.branch_sum_norms) when there is no shared
+        and no identity expert."""
         T = h.shape[0]
         logits = None
         if T >= self.ROUTE_PRODUCT_MIN_TOKENS:
@@ -137,7 +146,8 @@ class RoutedExperts(nn.Module):
         experts, weights, sg = ops.moe_route(h, self.router.data, self.correction.data,
                                              None if self.shared_gate is None else self.shared_gate.data, self.top, logits,
                                              None if self.router_bias is None else self.router_bias.data,
-                                             self.score, self.renormalize)
+                                             self.score, self.renormalize, self.groups, self.keep_groups,
+                                             self.weight_scale)
         if self.num_experts:
             row_scale = None
             if self.weight_input:
@@ -158,6 +168,12 @@ class RoutedExperts(nn.Module):
         else:   # identity experts only
             pair_row = torch.full((T, self.top), -1, dtype=torch.int32, device=h.device)
             y = torch.zeros((1, self.width), dtype=torch.float32, device=h.device)
+        return y, pair_row, weights, sg
+
+    def forward(self, h: torch.Tensor) -> torch.Tensor:
+        """h [T, width] in the activation dtype -> fp32 [T, width]."""
+        T = h.shape[0]
+        y, pair_row, weights, sg = self.rows(h)
         shared_y = None
         if self.shared_ff:
             su = torch.mm(h, self.shared_up.data.t())
