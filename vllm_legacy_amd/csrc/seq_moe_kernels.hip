@@ -45,7 +45,7 @@ __global__ __launch_bounds__(256) void moe_route_kernel(
     const float* __restrict__ correction,
     const float* __restrict__ shared_gate_w, int* __restrict__ experts, float* __restrict__ weights,
     float* __restrict__ shared_gate, int width, int routed, int top, int score, int renormalize,
-    int groups, int keep_groups, float weight_scale) {
+    int groups, int keep_groups, float weight_scale, bool vec) {
   __shared__ float z[kMaxRouted + 1];
   __shared__ float group_best[kMaxRouted];
   __shared__ int group_open[kMaxRouted];
@@ -60,7 +60,28 @@ __global__ __launch_bounds__(256) void moe_route_kernel(
     for (int n = w; n < rows; n += 4) {
       const float* wr = n < routed ? router + (int64_t)n * width : shared_gate_w;
       float dot = 0.f;
-      for (int c = lane; c < width; c += kWave) dot += wr[c] * S::to_f32(hr[c]);
+      if (vec) {                     // eight values per access, several accesses in flight
+#pragma unroll 4
+        for (int c = 8 * lane; c < width; c += 8 * kWave) {
+          const f32x4 w0 = *reinterpret_cast<const f32x4*>(wr + c), w1 = *reinterpret_cast<const f32x4*>(wr + c + 4);
+          float x[8];
+          if constexpr (sizeof(typename S::T) == 2) {
+            const u32x4 hv = *reinterpret_cast<const u32x4*>(hr + c);
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+              x[2 * e] = lo16<S>(hv[e]);
+              x[2 * e + 1] = hi16<S>(hv[e]);
+            }
+          } else {
+#pragma unroll
+            for (int e = 0; e < 8; ++e) x[e] = hr[c + e];
+          }
+#pragma unroll
+          for (int e = 0; e < 4; ++e) dot += w0[e] * x[e] + w1[e] * x[4 + e];
+        }
+      } else {
+        for (int c = lane; c < width; c += kWave) dot += wr[c] * S::to_f32(hr[c]);
+      }
       dot = wave_sum(dot);
       if (lane == 0) z[n] = dot + (bias != nullptr && n < routed ? bias[n] : 0.f);
     }
@@ -569,12 +590,15 @@ extern "C" int vla_seq_moe_route(const void* h, int64_t h_stride, const float* r
       (logits ? logits_stride < routed + (gated ? 1 : 0)
               : (!h || !router || h_stride < width || (gated && !shared_gate_weight))))
     return VLA_ERR_ARG;
+  const int size = dtype == VLA_F32 ? 4 : 2;
+  const bool vec = !logits && width % 8 == 0 && (uintptr_t)h % (8 * size) == 0 && h_stride % 8 == 0 &&
+                   (uintptr_t)router % 16 == 0 && (uintptr_t)shared_gate_weight % 16 == 0;
   return with_dtype(dtype, [&](auto s) {
     using S = decltype(s);
     moe_route_kernel<S><<<num_tokens, 256, 0, (hipStream_t)stream>>>(
         (const typename S::T*)h, h_stride, router, logits, logits_stride, bias, correction,
         shared_gate_weight, experts, weights, shared_gate, width, routed, top, score, renormalize, groups,
-        keep_groups, weight_scale);
+        keep_groups, weight_scale, vec);
     VLA_SEQ_HIP_CHECK(hipGetLastError());
     return VLA_OK;
   });
