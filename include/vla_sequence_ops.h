@@ -232,7 +232,7 @@ int vla_seq_rotary_kv_write(void* q, int64_t q_stride, const void* k, int64_t k_
  *   o = sum_j w_j v_j,  w_j = e^(s_j) / (sum_k e^(s_k) + e^(sinks[h]))   (sinks fp32 [heads]; null: softmax);  out_inv_freq given: pair m of o turns by -p * out_inv_freq[m]
  *   out = dtype(o * sigmoid(gate[t, h]))                      (gate null: no gate)
  * in fp32; the step's own keys and values must be in the caches already.  gate holds one number
- * per (token, head) with row stride gate_stride. */
+ * per (token, head) with row stride gate_stride.  dim and vdim up to 512. */
 int vla_seq_kv_attention(void* out, int64_t out_stride, const void* q, int64_t q_stride,
                          const void* gate, int64_t gate_stride, const void* key_cache,
                          const void* value_cache, const int* block_tables, int max_blocks,
@@ -244,11 +244,12 @@ int vla_seq_kv_attention(void* out, int64_t out_stride, const void* q, int64_t q
 
 /* The same attention for 16-bit activations, tiled over runs of 32 query rows of a sequence on
  * the matrix cores: rows query_start_loc[b] .. query_start_loc[b + 1] - 1 of sequence b sit at
- * positions context_lens[b] ...  dim and vdim must be multiples of 32, at most 128
- * (vla_seq_kv_attention_tiles_supported); query rows and cache rows must be 8-byte aligned.
+ * positions context_lens[b] ...  dim must be a multiple of 32 up to 128, vdim one up to 512 (values of
+ * more than 128 dims in slices, a launch each; up to 128 with out_inv_freq)
+ * (vla_seq_kv_attention_tiles_supported; turned: with out_inv_freq); query rows and cache rows must be 8-byte aligned.
  * vla_seq_kv_attention takes single rows of such shapes to the matrix cores by itself;
  * vla_seq_set_kv_attention_kernel(1) keeps both off them (tests run both), 0 is the default. */
-int vla_seq_kv_attention_tiles_supported(int dim, int vdim, int dtype);
+int vla_seq_kv_attention_tiles_supported(int dim, int vdim, int turned, int dtype);
 int vla_seq_kv_attention_tiles(void* out, int64_t out_stride, const void* q, int64_t q_stride,
                                const void* gate, int64_t gate_stride, const void* key_cache,
                                const void* value_cache, const int* block_tables, int max_blocks,

@@ -488,7 +488,8 @@ def test_head_norms_with_a_factor_per_head(dtype, n, groups):
 
 # ----------------------------------------------------------------------------- windowed attention
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
-@pytest.mark.parametrize("shape", [(4, 2, 16, 24, 9, 8), (8, 4, 96, 192, 40, 24), (3, 1, 10, 7, 33, 10), (8, 2, 64, 128, 64, 32)])
+@pytest.mark.parametrize("shape", [(4, 2, 16, 24, 9, 8), (8, 4, 96, 192, 40, 24), (3, 1, 10, 7, 33, 10), (8, 2, 64, 128, 64, 32),
+                                   (2, 1, 32, 320, 20, 8), (2, 2, 300, 400, 17, 16), (6, 3, 128, 160, 50, 64)])
 def test_window_edges_by_one_planted_key(dtype, shape):
     """One key matches one query through an unrotated (or, where all turn, the slowest) dimension; it is
     seen at a distance of window - 1 and not at a distance of window, in a prompt, in portions and

@@ -119,7 +119,7 @@ def seq_lib():
                                               i, i, i, i, i, p, p, f, p, i64, p, i, p]
         L.vla_seq_kv_attention.argtypes = [p, i64, p, i64, p, i64, p, p, p, i, p, p, p, i, i, i, i, i,
                                            i, i, i, i, f, i, i, f, i, p, p]
-        L.vla_seq_kv_attention_tiles_supported.argtypes = [i, i, i]
+        L.vla_seq_kv_attention_tiles_supported.argtypes = [i, i, i, i]
         L.vla_seq_kv_attention_tiles.argtypes = [p, i64, p, i64, p, i64, p, p, p, i, p, p, p, i, i, i,
                                                  i, i, i, i, i, i, i, f, i, i, f, i, p, p]
         L.vla_seq_set_kv_attention_kernel.argtypes = [i]

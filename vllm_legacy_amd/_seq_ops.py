@@ -483,9 +483,10 @@ def set_kv_attention_kernel(mode: int) -> None:
     seq_check(_lib.seq_lib().vla_seq_set_kv_attention_kernel(mode), "set_kv_attention_kernel")
 
 
-def kv_attention_tiles_supported(q: torch.Tensor, head_dim: int, value_dim: int) -> bool:
-    """Whether the matrix-core kernel for runs of query rows takes this query tensor."""
-    return bool(_lib.seq_lib().vla_seq_kv_attention_tiles_supported(head_dim, value_dim, _dt(q.dtype))) and \
+def kv_attention_tiles_supported(q: torch.Tensor, head_dim: int, value_dim: int, turned: bool = False) -> bool:
+    """Whether the matrix-core kernel for runs of query rows takes this query tensor (turned: outputs are
+    turned back by their position)."""
+    return bool(_lib.seq_lib().vla_seq_kv_attention_tiles_supported(head_dim, value_dim, int(turned), _dt(q.dtype))) and \
         q.data_ptr() % 16 == 0 and (q.stride(0) * q.element_size()) % 16 == 0
 
 

@@ -17,9 +17,9 @@ sigmoid of one number per (token, head); forward's `v_other` / `v_blend` cache
 (1 - v_blend) v + v_blend v_other instead of v (values blended with another layer's values of the
 same tokens).  Every parameter is a constructor argument.  Prompts, portions of prompts and decode steps are one case: the step's keys and values
 are written to the caches, then every row reads from there (csrc/seq_kv_attention.hip: matrix-core
-kernels for 16-bit models whose head sizes are multiples of 32 -- tiles of 32 rows for runs of
-rows, all heads of a KV group at once for single rows -- and an fp32 kernel for any dtype and head
-size).
+kernels for 16-bit models whose head sizes are multiples of 32 (values wider than 128 in slices) --
+tiles of 32 rows for runs of rows, all heads of a KV group at once for single rows -- and an fp32 kernel
+for any dtype and head sizes up to 512).
 """
 from typing import Optional, Tuple
 
@@ -90,7 +90,8 @@ class RotaryKVAttention(nn.Module):
                             None if self.k_norm is None else self.k_norm.data, self.norm_eps, v_other, v_blend,
                             self.norm_heads)
         if batch.max_query_len >= self.TILE_MIN_QUERY and \
-                ops.kv_attention_tiles_supported(q, self.head_dim, self.value_dim):
+                ops.kv_attention_tiles_supported(q, self.head_dim, self.value_dim,
+                                                 self.value_inv_freq is not None):
             # a step with runs of rows (prompts, portions): 32-row tiles on the matrix cores
             ops.kv_attention_tiles(out, q, gate, key_cache, value_cache, batch.block_tables,
                                    batch.query_start_loc, batch.context_lens, batch.max_query_len,

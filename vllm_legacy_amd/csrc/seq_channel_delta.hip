@@ -372,19 +372,15 @@ __global__ __launch_bounds__(256) void delta_walk_kernel(ChannelDelta a) {
     const int row = i * kRows + 4 * g + w;
     if (row < run && col < V) a.o[((int64_t)(t_begin + row) * a.heads + h) * V + col] = o;
   };
-  // AHEAD blocks in turn: while one is worked on, the others are on their way
-  constexpr int AHEAD = 2;
-  Block f[AHEAD];
-#pragma unroll
-  for (int e = 0; e < AHEAD - 1; ++e) fetch(f[e], min(e, blocks - 1));
-  for (int i0 = 0; i0 < blocks; i0 += AHEAD) {
-#pragma unroll
-    for (int e = 0; e < AHEAD; ++e) {
-      const int i = i0 + e;
-      if (i >= blocks) break;
-      fetch(f[(e + AHEAD - 1) % AHEAD], min(i + AHEAD - 1, blocks - 1));
-      advance(f[e], i);
-    }
+  // two blocks in turn, so that one is asked for while the other is worked on
+  Block f0, f1;
+  fetch(f0, 0);
+  for (int i = 0; i < blocks; i += 2) {
+    fetch(f1, min(i + 1, blocks - 1));
+    advance(f0, i);
+    if (i + 1 >= blocks) break;
+    fetch(f0, min(i + 2, blocks - 1));
+    advance(f1, i + 1);
   }
   if (col < V) {
 #pragma unroll

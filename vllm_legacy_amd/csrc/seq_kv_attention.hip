@@ -29,8 +29,7 @@ namespace vla {
 namespace seq {
 namespace {
 
-constexpr int kMaxDim = 256;
-constexpr int kAccum = kMaxDim / kWave;
+constexpr int kMaxDim = 512;
 constexpr int kHeadsPerGroup = 4;
 
 // the pair (a, b) turned by angle: (a cos - b sin, b cos + a sin)
@@ -236,7 +235,7 @@ __device__ __forceinline__ void write_head_output(typename S::T* __restrict__ or
   }
 }
 
-template <class S>
+template <class S, int kAccum>    // kAccum values per lane: rows of up to 64 kAccum
 __global__ __launch_bounds__(kWave* kHeadsPerGroup) void kv_attention_kernel(
     typename S::T* __restrict__ out, int64_t out_stride, const typename S::T* __restrict__ q,
     int64_t q_stride, const typename S::T* __restrict__ gate, int64_t gate_stride,
@@ -245,7 +244,7 @@ __global__ __launch_bounds__(kWave* kHeadsPerGroup) void kv_attention_kernel(
     const int64_t* __restrict__ positions, const float* __restrict__ out_inv_freq, int interleaved,
     int heads, int kv_heads, int dim, int vdim, int block_size, int num_blocks, int window,
     float scale, int keep_first, float softcap, int chunk, const float* __restrict__ sinks) {
-  __shared__ float q_lds[kHeadsPerGroup][kMaxDim];
+  __shared__ float q_lds[kHeadsPerGroup][kWave * kAccum];
   __shared__ float p_lds[kHeadsPerGroup][kWave];
   const int lane = threadIdx.x & 63, w = threadIdx.x >> 6;
   const int t = blockIdx.x;
@@ -464,7 +463,7 @@ __global__ __launch_bounds__(256, 2) void kv_attention_tile_kernel(
     const int* __restrict__ block_tables, int max_blocks, const int* __restrict__ query_start_loc,
     const int* __restrict__ context_lens, const float* __restrict__ out_inv_freq, int interleaved,
     int heads, int kv_heads, int block_size, int num_blocks, int window, float scale, int head_waves,
-    int keep_first, float softcap, int chunk, const float* __restrict__ sinks) {
+    int keep_first, float softcap, int chunk, const float* __restrict__ sinks, int v_row, int v_first) {
   using T = typename S::T;
   using M = Mfma16<S>;
   constexpr int D = 32 * DB, VD = 32 * VB;
@@ -557,7 +556,7 @@ __global__ __launch_bounds__(256, 2) void kv_attention_tile_kernel(
       const int i = tid + 256 * u;
       const int r = i / (VD / 8), v = i % (VD / 8);
       const long long row = rows_lds[buf][r];
-      const u32x4 got = *reinterpret_cast<const u32x4*>(value_cache + (row >= 0 ? row * VD + 8 * v : 0));
+      const u32x4 got = *reinterpret_cast<const u32x4*>(value_cache + (row >= 0 ? row * v_row + v_first + 8 * v : 0));
       xv[u] = row >= 0 ? got : u32x4{0u, 0u, 0u, 0u};
     }
   };
@@ -699,7 +698,7 @@ __global__ __launch_bounds__(256, 2) void kv_attention_tile_kernel(
   for (int n = 0; n < VB; ++n)
 #pragma unroll
     for (int i = 0; i < 16; ++i)
-      out[(int64_t)(t0 + c) * out_stride + (int64_t)h * VD + out_dim(n, i, hf)] = S::from_f32(o[n][i] * gv);
+      out[(int64_t)(t0 + c) * out_stride + (int64_t)h * v_row + v_first + out_dim(n, i, hf)] = S::from_f32(o[n][i] * gv);
 }
 
 // kv_attention_heads_kernel<S, DB, VB>: single rows (decode steps).  One workgroup per (row, KV
@@ -717,7 +716,8 @@ __global__ __launch_bounds__(64 * kRowWaves) void kv_attention_heads_kernel(
     const int* __restrict__ block_tables, int max_blocks, const int* __restrict__ token_seq,
     const int64_t* __restrict__ positions, const float* __restrict__ out_inv_freq, int interleaved,
     int heads, int kv_heads, int block_size, int num_blocks, int window, float scale,
-    int merge_heads, int keep_first, float softcap, int chunk, const float* __restrict__ sinks) {
+    int merge_heads, int keep_first, float softcap, int chunk, const float* __restrict__ sinks,
+    int v_row, int v_first) {
   using T = typename S::T;
   using M = Mfma8<S>;
   constexpr int D = 32 * DB, VD = 32 * VB;
@@ -787,7 +787,7 @@ __global__ __launch_bounds__(64 * kRowWaves) void kv_attention_heads_kernel(
       const int i = lane + kWave * u;
       const int r = i / (VD / 4), v = i % (VD / 4);
       const long long rb = __shfl(row, r, 64);
-      const u32x2 got = *reinterpret_cast<const u32x2*>(value_cache + (rb >= 0 ? rb * VD + 4 * v : 0));
+      const u32x2 got = *reinterpret_cast<const u32x2*>(value_cache + (rb >= 0 ? rb * v_row + v_first + 4 * v : 0));
       xv[u] = rb >= 0 ? got : u32x2{0u, 0u};
     }
   };
@@ -903,7 +903,7 @@ __global__ __launch_bounds__(64 * kRowWaves) void kv_attention_heads_kernel(
       val = is_a ? val * c2 + ov * s : val * c2 - ov * s;
     }
     if (gate != nullptr) val *= 1.f / (1.f + expf(-S::to_f32(gate[(int64_t)t * gate_stride + h0 + hh])));
-    out[(int64_t)t * out_stride + (int64_t)(h0 + hh) * VD + d] = S::from_f32(val);
+    out[(int64_t)t * out_stride + (int64_t)(h0 + hh) * v_row + v_first + d] = S::from_f32(val);
   }
 }
 
@@ -915,7 +915,7 @@ int launch_heads_one(dim3 grid, hipStream_t stream, typename S::T* out, int64_t 
                      const int* token_seq, const int64_t* positions, const float* out_inv_freq,
                      int interleaved, int heads, int kv_heads, int block_size, int num_blocks,
                      int window, float scale, int keep_first, float softcap, int chunk,
-                     const float* sinks) {
+                     const float* sinks, int v_row, int v_first) {
   constexpr int D = 32 * DB, VD = 32 * VB;
   const int group = heads / kv_heads;
   const int merge_heads = group < 32 ? group : 32;
@@ -933,7 +933,7 @@ int launch_heads_one(dim3 grid, hipStream_t stream, typename S::T* out, int64_t 
   kv_attention_heads_kernel<S, DB, VB><<<grid, 64 * kRowWaves, lds, stream>>>(
       out, out_stride, q, q_stride, gate, gate_stride, key_cache, value_cache, block_tables,
       max_blocks, token_seq, positions, out_inv_freq, interleaved, heads, kv_heads, block_size,
-      num_blocks, window, scale, merge_heads, keep_first, softcap, chunk, sinks);
+      num_blocks, window, scale, merge_heads, keep_first, softcap, chunk, sinks, v_row, v_first);
   VLA_SEQ_HIP_CHECK(hipGetLastError());
   return VLA_OK;
 }
@@ -946,11 +946,11 @@ int launch_tiles_one(dim3 grid, hipStream_t stream, typename S::T* out, int64_t 
                      const int* qsl, const int* ctx, const float* out_inv_freq, int interleaved,
                      int heads, int kv_heads, int block_size, int num_blocks, int window,
                      float scale, int head_waves, int keep_first, float softcap, int chunk,
-                     const float* sinks) {
+                     const float* sinks, int v_row, int v_first) {
   kv_attention_tile_kernel<S, DB, VB><<<grid, 256, 0, stream>>>(
       out, out_stride, q, q_stride, gate, gate_stride, key_cache, value_cache, block_tables,
       max_blocks, qsl, ctx, out_inv_freq, interleaved, heads, kv_heads, block_size, num_blocks,
-      window, scale, head_waves, keep_first, softcap, chunk, sinks);
+      window, scale, head_waves, keep_first, softcap, chunk, sinks, v_row, v_first);
   VLA_SEQ_HIP_CHECK(hipGetLastError());
   return VLA_OK;
 }
@@ -986,8 +986,23 @@ int launch_tiles(int db, int vb, A... a) {
   VLA_KV_BY_SIZE(launch_tiles_one, S, db, vb, a...)
 }
 
-bool mfma_sizes(int dim, int vdim) {
-  return dim % 32 == 0 && dim >= 32 && dim <= 128 && vdim % 32 == 0 && vdim >= 32 && vdim <= 128;
+// Values of more than 128 dims go in slices: each a launch that forms the same weights again and sums
+// its columns (values that turn back pair columns across slices and do not).
+constexpr int kSliceBlocks = 4;
+bool mfma_sizes(int dim, int vdim, bool turned) {
+  return dim % 32 == 0 && dim >= 32 && dim <= 128 && vdim % 32 == 0 && vdim >= 32 &&
+         vdim <= (turned ? 32 * kSliceBlocks : kMaxDim);
+}
+// f(vdim / 32 of the slice, first column) for slices of about equal size
+template <class F>
+int by_value_slices(int vdim, F&& f) {
+  const int blocks = vdim / 32, slices = (blocks + kSliceBlocks - 1) / kSliceBlocks;
+  for (int s = 0; s < slices; ++s) {
+    const int first = blocks * s / slices, end = blocks * (s + 1) / slices;
+    const int rc = f(end - first, 32 * first);
+    if (rc != VLA_OK) return rc;
+  }
+  return VLA_OK;
 }
 
 }  // namespace
@@ -1052,26 +1067,33 @@ extern "C" int vla_seq_kv_attention(void* out, int64_t out_stride, const void* q
     using T = typename S::T;
     if constexpr (sizeof(T) == 2) {
       // 16-bit rows on the matrix cores when the head sizes and the alignment allow
-      if (g_kv_kernel.load(std::memory_order_relaxed) == 0 && mfma_sizes(dim, vdim) &&
+      if (g_kv_kernel.load(std::memory_order_relaxed) == 0 && mfma_sizes(dim, vdim, out_inv_freq != nullptr) &&
           ((uintptr_t)q % 8) == 0 && ((q_stride * 2) % 8) == 0 && ((uintptr_t)key_cache % 8) == 0 &&
           ((uintptr_t)value_cache % 8) == 0) {
         const int group = heads / kv_heads;
         const dim3 grid(num_tokens, kv_heads * ((group + 31) / 32));
-        const int rc = launch_heads<S>(dim / 32, vdim / 32, grid, (hipStream_t)stream, (T*)out, out_stride,
-                                       (const T*)q, q_stride, (const T*)gate, gate_stride,
-                                       (const T*)key_cache, (const T*)value_cache, block_tables,
-                                       max_blocks, token_seq, positions, out_inv_freq, interleaved,
-                                       heads, kv_heads, block_size, num_blocks, window, scale,
-                                       keep_first, softcap, chunk, sinks);
+        const int rc = by_value_slices(vdim, [&](int vb, int v_first) {
+          return launch_heads<S>(dim / 32, vb, grid, (hipStream_t)stream, (T*)out, out_stride, (const T*)q,
+                                 q_stride, (const T*)gate, gate_stride, (const T*)key_cache,
+                                 (const T*)value_cache, block_tables, max_blocks, token_seq, positions,
+                                 out_inv_freq, interleaved, heads, kv_heads, block_size, num_blocks,
+                                 window, scale, keep_first, softcap, chunk, sinks, vdim, v_first);
+        });
         if (rc != VLA_ERR_HEAD_SIZE) return rc;
       }
     }
     const dim3 grid(num_tokens, (heads + kHeadsPerGroup - 1) / kHeadsPerGroup);
-    kv_attention_kernel<S><<<grid, kWave * kHeadsPerGroup, 0, (hipStream_t)stream>>>(
-        (T*)out, out_stride, (const T*)q, q_stride, (const T*)gate, gate_stride,
-        (const T*)key_cache, (const T*)value_cache, block_tables, max_blocks, token_seq, positions,
-        out_inv_freq, interleaved, heads, kv_heads, dim, vdim, block_size, num_blocks, window, scale,
-        keep_first, softcap, chunk, sinks);
+    auto plain = [&](auto kernel) {
+      kernel<<<grid, kWave * kHeadsPerGroup, 0, (hipStream_t)stream>>>(
+          (T*)out, out_stride, (const T*)q, q_stride, (const T*)gate, gate_stride, (const T*)key_cache,
+          (const T*)value_cache, block_tables, max_blocks, token_seq, positions, out_inv_freq,
+          interleaved, heads, kv_heads, dim, vdim, block_size, num_blocks, window, scale, keep_first,
+          softcap, chunk, sinks);
+    };
+    if (dim <= 256 && vdim <= 256)
+      plain(kv_attention_kernel<S, 4>);
+    else
+      plain(kv_attention_kernel<S, kMaxDim / kWave>);
     VLA_SEQ_HIP_CHECK(hipGetLastError());
     return VLA_OK;
   });
@@ -1084,8 +1106,8 @@ extern "C" int vla_seq_set_kv_attention_kernel(int mode) {
   return VLA_OK;
 }
 
-extern "C" int vla_seq_kv_attention_tiles_supported(int dim, int vdim, int dtype) {
-  return (dtype == VLA_F16 || dtype == VLA_BF16) && mfma_sizes(dim, vdim) &&
+extern "C" int vla_seq_kv_attention_tiles_supported(int dim, int vdim, int turned, int dtype) {
+  return (dtype == VLA_F16 || dtype == VLA_BF16) && mfma_sizes(dim, vdim, turned != 0) &&
          g_kv_kernel.load(std::memory_order_relaxed) == 0;
 }
 
@@ -1105,7 +1127,8 @@ extern "C" int vla_seq_kv_attention_tiles(
       out_stride < (int64_t)heads * vdim || q_stride < (int64_t)heads * dim ||
       (gate && gate_stride < heads))
     return VLA_ERR_ARG;
-  if ((dtype != VLA_F16 && dtype != VLA_BF16) || !mfma_sizes(dim, vdim)) return VLA_ERR_HEAD_SIZE;
+  if ((dtype != VLA_F16 && dtype != VLA_BF16) || !mfma_sizes(dim, vdim, out_inv_freq != nullptr))
+    return VLA_ERR_HEAD_SIZE;
   // 8-byte fragment loads: query rows and cache rows must allow them
   if (((uintptr_t)q % 8) || ((q_stride * 2) % 8) || ((uintptr_t)key_cache % 8) ||
       ((uintptr_t)value_cache % 8))
@@ -1119,17 +1142,16 @@ extern "C" int vla_seq_kv_attention_tiles(
   const int tile_rows = kTile * (4 / head_waves);
   const dim3 grid((max_query_len + tile_rows - 1) / tile_rows,
                   kv_heads * ((group + head_waves - 1) / head_waves), num_seqs);
-  if (dtype == VLA_BF16)
-    return launch_tiles<BF16>(dim / 32, vdim / 32, grid, (hipStream_t)stream, (__bf16*)out, out_stride,
-                              (const __bf16*)q, q_stride, (const __bf16*)gate, gate_stride,
-                              (const __bf16*)key_cache, (const __bf16*)value_cache, block_tables,
-                              max_blocks, query_start_loc, context_lens, out_inv_freq, interleaved,
-                              heads, kv_heads, block_size, num_blocks, window, scale, head_waves,
-                              keep_first, softcap, chunk, sinks);
-  return launch_tiles<F16>(dim / 32, vdim / 32, grid, (hipStream_t)stream, (_Float16*)out, out_stride,
-                           (const _Float16*)q, q_stride, (const _Float16*)gate, gate_stride,
-                           (const _Float16*)key_cache, (const _Float16*)value_cache, block_tables,
-                           max_blocks, query_start_loc, context_lens, out_inv_freq, interleaved, heads,
-                           kv_heads, block_size, num_blocks, window, scale, head_waves, keep_first,
-                           softcap, chunk, sinks);
+  auto go = [&](auto tag) {
+    using S = decltype(tag);
+    using T = typename S::T;
+    return by_value_slices(vdim, [&](int vb, int v_first) {
+      return launch_tiles<S>(dim / 32, vb, grid, (hipStream_t)stream, (T*)out, out_stride, (const T*)q, q_stride,
+                             (const T*)gate, gate_stride, (const T*)key_cache, (const T*)value_cache,
+                             block_tables, max_blocks, query_start_loc, context_lens, out_inv_freq,
+                             interleaved, heads, kv_heads, block_size, num_blocks, window, scale,
+                             head_waves, keep_first, softcap, chunk, sinks, vdim, v_first);
+    });
+  };
+  return dtype == VLA_BF16 ? go(BF16{}) : go(F16{});
 }
