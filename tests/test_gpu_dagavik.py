@@ -342,7 +342,7 @@ def test_channel_delta_layer(dtype, shape):
 
 
 # ----------------------------------------------------------------------------- matrix memory
-MEMORY_SHAPES = [(2, 8, 8), (4, 16, 24), (3, 10, 7), (4, 32, 64), (2, 128, 128), (1, 96, 200), (2, 20, 300), (1, 160, 16), (5, 1, 1)]
+MEMORY_SHAPES = [(2, 8, 8), (4, 16, 24), (3, 10, 7), (3, 32, 96), (2, 128, 128), (1, 96, 200), (2, 20, 300), (1, 160, 16), (5, 1, 1)]
 
 
 def memory_inputs(n, shape, seed, dtype, spread=3.0):
@@ -488,7 +488,7 @@ def test_head_norms_with_a_factor_per_head(dtype, n, groups):
 
 # ----------------------------------------------------------------------------- windowed attention
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
-@pytest.mark.parametrize("shape", [(4, 2, 16, 24, 9, 8), (8, 4, 96, 192, 40, 24), (3, 1, 10, 7, 33, 10), (8, 2, 64, 128, 64, 32),
+@pytest.mark.parametrize("shape", [(4, 2, 16, 24, 9, 8), (6, 2, 64, 192, 40, 16), (3, 1, 10, 7, 33, 10), (8, 2, 64, 128, 64, 32),
                                    (2, 1, 32, 320, 20, 8), (2, 2, 300, 400, 17, 16), (6, 3, 128, 160, 50, 64)])
 def test_window_edges_by_one_planted_key(dtype, shape):
     """One key matches one query through an unrotated (or, where all turn, the slowest) dimension; it is
@@ -611,7 +611,7 @@ def test_latent_attention_finds_one_far_key(dtype):
 
 
 # ----------------------------------------------------------------------------- experts
-@pytest.mark.parametrize("experts,groups,keep,top", [(12, 3, 2, 4), (8, 8, 3, 3), (6, 1, 1, 2), (9, 3, 1, 3), (70, 7, 4, 5),
+@pytest.mark.parametrize("experts,groups,keep,top", [(15, 5, 2, 4), (8, 8, 3, 3), (6, 1, 1, 2), (9, 3, 1, 3), (70, 7, 4, 5),
                                                      (128, 64, 2, 4), (5, 5, 5, 5), (256, 8, 4, 8)])
 def test_router_among_groups(experts, groups, keep, top):
     """Only experts of the best groups can be chosen; weights are the scores over all experts times the
@@ -625,9 +625,9 @@ def test_router_among_groups(experts, groups, keep, top):
         idx = torch.stack([R.choose(s[i], top, groups, keep) for i in range(T)])
         for logits in (None, z.float().to(DEV)):
             e, w, _ = ops.moe_route(h.to(DEV), router.to(DEV), None, None, top, logits, renormalize=False, groups=groups,
-                                    keep_groups=keep, weight_scale=2.5)
+                                    keep_groups=keep, weight_scale=1.9)
             assert torch.equal(e.cpu().long(), idx)
-            close(w, 2.5 * s.gather(1, idx), 3e-6)
+            close(w, 1.9 * s.gather(1, idx), 3e-6)
     if keep < groups and keep * (experts // groups) > top:
         assert not torch.equal(idx, torch.topk(s, top, -1).indices)
 
