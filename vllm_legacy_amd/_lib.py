@@ -41,9 +41,10 @@ EXPORTS = [
 ]
 
 
-def build(jobs: int = 8) -> str:
-    """Compile the HIP sources for gfx950 (hipcc cross-compiles without a GPU): both libraries."""
-    subprocess.check_call(["make", "-s", "-j%d" % jobs, "-C", CSRC])
+def build(jobs: int = 8, everything: bool = False) -> str:
+    """Compile the HIP sources for gfx950 (hipcc cross-compiles without a GPU): both libraries, what
+    changed since the last build or (`everything`) all of it."""
+    subprocess.check_call(["make", "-s", "-j%d" % jobs] + (["-B"] if everything else []) + ["-C", CSRC])
     return LIB_PATH
 
 
